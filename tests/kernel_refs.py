@@ -67,12 +67,15 @@ class TorchOps:
             else self.linear(h, weight, out_dtype)
         return out, resid
 
-    def linear_silu_mul(self, x, weight, out_dtype):
-        return self.silu_mul(self.linear(x, weight, out_dtype))
+    def linear_silu_mul(self, x, weight, out_dtype, limit=None):
+        return self.silu_mul(self.linear(x, weight, out_dtype), limit)
 
-    def silu_mul(self, gate_up):
+    def silu_mul(self, gate_up, limit=None):
         inner = gate_up.shape[-1] // 2
         g, u = gate_up[:, :inner].float(), gate_up[:, inner:].float()
+        if limit is not None:
+            g, u = torch.clamp(g, max=limit), torch.clamp(u, -limit, limit)
+            return (g * torch.sigmoid(1.702 * g) * (u + 1.0)).to(gate_up.dtype)
         return (g * torch.sigmoid(g) * u).to(gate_up.dtype)
 
     # ---------------------------------------------------------------- q/k preparation
@@ -145,8 +148,9 @@ class TorchOps:
     # ---------------------------------------------------------------- attention
     def paged_attention(self, q, batch, table, cache, *, num_heads, num_kv_heads, head_dim,
                         scale, window, only=None, sink=None, chunk=None, softcap=None,
-                        slopes=None, q_temp=None):
-        """`only`: compute just these flat tokens (a test's choice; the other rows of the
+                        slopes=None, q_temp=None, keep_first=0):
+        """`keep_first`: the first so many keys are seen whatever window or chunk says.
+        `only`: compute just these flat tokens (a test's choice; the other rows of the
         result are left unset).  `chunk`: a query sees the keys of its own stretch of that
         many positions; `softcap`: s <- cap tanh(s / cap); `slopes` [heads]: slope x distance
         comes off a score; `q_temp` (coef, every): the query's factor 1 + coef ln(floor((p +
@@ -163,7 +167,8 @@ class TorchOps:
                 lo = max(lo, p // chunk * chunk)
             temp = 1.0 if q_temp is None else \
                 1.0 + q_temp[0] * math.log((p + 1) // q_temp[1] + 1)
-            keys = torch.arange(lo, p + 1, device=q.device)
+            keys = torch.cat([torch.arange(min(keep_first, lo), device=q.device),
+                              torch.arange(lo, p + 1, device=q.device)])
             pages = table[b, keys // P].long()
             if (pages < 0).any():
                 raise RuntimeError("attention reads a position whose page was given back")
@@ -215,6 +220,18 @@ class TorchOps:
 
     def postnorm_add(self, resid, delta, post_w, eps):
         resid.add_(self._unit(delta.float(), eps) * post_w.float())
+
+    def postnorm_add_rows(self, resid, delta, post_w, eps, out_dtype):
+        self.postnorm_add(resid, delta, post_w, eps)
+        return self.stream_rows(resid, out_dtype)
+
+    def stream_rows(self, resid, out_dtype):
+        return resid if out_dtype == torch.float32 else resid.to(out_dtype)
+
+    def token_gate(self, z, table, ids, col, out_dtype):
+        z = z.float()
+        gate = 0.5 * z * (1.0 + torch.tanh(0.7978845608028654 * (z + 0.044715 * z ** 3)))
+        return (gate * table[ids.long(), col:col + z.shape[1]].float()).to(out_dtype)
 
     def postnorm_add_norm(self, resid, delta, post_w, post_eps, norm_w, norm_eps, out_dtype):
         self.postnorm_add(resid, delta, post_w, post_eps)
@@ -484,9 +501,26 @@ class TorchOps:
         cache.k_pages[page, pos % P] = torch.cat([c, kr], dim=-1).to(cache.k_pages.dtype)
         return cq.to(out_dtype)
 
+    def latent_rows(self, rows, batch, table, cache, *, heads, own, kv_rank, rot_dim, kv_norm, eps,
+                    freqs, rot_dims):
+        T, dl = rows.shape[0], kv_rank + rot_dim
+        if own:
+            P = cache.page_size
+            c = self._unit(rows[:, heads * dl:heads * dl + kv_rank], eps) * kv_norm.float()
+            kr = self._rotate_pairs(rows[:, heads * dl + kv_rank:], batch.positions, freqs, rot_dims)
+            pos = batch.positions.long()
+            page = table[batch.entry_of_token.long(), pos // P].long()
+            if (page < 0).any():
+                raise RuntimeError("store to a position whose page was given back")
+            cache.k_pages[page, pos % P] = torch.cat([c, kr], dim=-1).to(cache.k_pages.dtype)
+        q = rows[:, :heads * dl].clone().view(T, heads, dl)
+        q[..., kv_rank:] = self._rotate_pairs(q[..., kv_rank:].clone(), batch.positions, freqs, rot_dims)
+        rows[:, :heads * dl] = q.reshape(T, heads * dl)
+
     def latent_attention(self, qa, batch, table, cache, *, heads, kv_rank, rot_dim, scale,
-                         window, out_dtype=torch.float32):
+                         window, out_dtype=torch.float32, sink=None):
         T = qa.shape[0]
+        qa = qa.reshape(T, -1)[:, :heads * (kv_rank + rot_dim)].reshape(T, heads, kv_rank + rot_dim)
         P = cache.page_size
         out = torch.empty(T, heads, kv_rank, dtype=torch.float32, device=qa.device)
         for t in range(T):
@@ -498,7 +532,9 @@ class TorchOps:
                 raise RuntimeError("attention reads a position whose page was given back")
             kv = cache.k_pages[pages, keys % P].float()          # [n, kv_rank + rot_dim]
             s = (kv @ qa[t].float().T) * scale                   # [n, heads]
-            out[t] = torch.softmax(s, dim=0).T @ kv[:, :kv_rank]
+            if sink is not None:        # one more score in every denominator
+                s = torch.cat([s, sink.float().view(1, heads)])
+            out[t] = torch.softmax(s, dim=0).T[:, :kv.shape[0]] @ kv[:, :kv_rank]
         return out.to(out_dtype)
 
     # ---------------------------------------------------------------- sampling

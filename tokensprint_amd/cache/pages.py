@@ -133,7 +133,8 @@ class GroupLayout:
 
     `window` None: every earlier key stays; W: a query at position p sees keys
     p-W+1..p, so a page whose last position is below that for every coming query
-    is given back.
+    is given back, except the pages of the sequence's first `keep_first` keys, which every
+    query sees beside its window.
     """
 
     num_kv_heads: int
@@ -143,6 +144,7 @@ class GroupLayout:
     #: "kv": keys and values per head; "latent": one vector of `head_dim` elements per
     #: token that every head reads (`num_kv_heads` is 1)
     kind: str = "kv"
+    keep_first: int = 0
 
 
 @dataclass
@@ -153,7 +155,8 @@ class RequestCache:
     slot: int
     tables: list[list[int]]        # per group: logical page -> physical id, -1 = given back
     num_tokens: int = 0            # positions [0, num_tokens) are in the cache
-    released: list[int] = field(default_factory=list)   # per group: leading pages given back
+    #: per group: pages below this have been given back, but for the kept first ones
+    released: list[int] = field(default_factory=list)
     hashes: list[int] = field(default_factory=list)     # chained hash of every registered full page
 
 
@@ -278,6 +281,11 @@ class CacheManager:
             return 0
         return max(0, first_query_pos - window + 1) // self.page_size
 
+    def _first_released(self, rc: RequestCache, g: int) -> int:
+        """Index of the first page that a release has still to look at: behind what has been
+        given back and behind the pages that are kept for good."""
+        return max(rc.released[g], -(-self.groups[g].keep_first // self.page_size))
+
     def pages_needed(self, rc: RequestCache, new_len: int) -> list[int]:
         """Per group, free pages that extending to `new_len` tokens takes from the
         pool, counting the pages the window lets go first."""
@@ -285,7 +293,7 @@ class CacheManager:
         total = -(-new_len // P)
         out = []
         for g, table in enumerate(rc.tables):
-            released_now = sum(1 for i in range(rc.released[g],
+            released_now = sum(1 for i in range(self._first_released(rc, g),
                                                 min(self._first_kept_page(g, rc.num_tokens),
                                                     len(table))) if table[i] >= 0)
             out.append(max(0, total - len(table)) - released_now)
@@ -299,7 +307,7 @@ class CacheManager:
             if len(table) * P < new_len:
                 return False
             if self.groups[g].window is not None and \
-                    self._first_kept_page(g, rc.num_tokens) > rc.released[g]:
+                    self._first_kept_page(g, rc.num_tokens) > self._first_released(rc, g):
                 return False
         return True
 
@@ -358,7 +366,7 @@ class CacheManager:
         """Give back the pages no query at position >= rc.num_tokens can see."""
         for g, table in enumerate(rc.tables):
             keep_from = min(self._first_kept_page(g, rc.num_tokens), len(table))
-            for i in range(rc.released[g], keep_from):
+            for i in range(self._first_released(rc, g), keep_from):
                 if table[i] >= 0:
                     self.pools[g].give_back(table[i])
                     table[i] = -1

@@ -25,7 +25,8 @@ from tokensprint_amd.parts.base import PagedKVNeed, PagedLatentNeed, SlotStateNe
 
 
 def group_runs(needs) -> tuple[list[GroupLayout], dict[int, int]]:
-    """Group the runs that own a paged cache by (kv heads, head size, window, kind)."""
+    """Group the runs that own a paged cache by (kv heads, head size, window, kind, kept first
+    keys)."""
     keyed: dict[tuple, list[int]] = {}
     for r, need in enumerate(needs):
         paged = [n for n in flat_needs(need) if isinstance(n, (PagedKVNeed, PagedLatentNeed))]
@@ -33,12 +34,12 @@ def group_runs(needs) -> tuple[list[GroupLayout], dict[int, int]]:
             raise ValueError(f"run {r} asks for {len(paged)} paged caches; a run owns one")
         for n in paged:
             if isinstance(n, PagedKVNeed):
-                keyed.setdefault((n.num_kv_heads, n.head_dim, n.window, "kv"), []).append(r)
+                keyed.setdefault((n.num_kv_heads, n.head_dim, n.window, "kv", n.keep_first), []).append(r)
             else:
-                keyed.setdefault((1, n.dim, n.window, "latent"), []).append(r)
+                keyed.setdefault((1, n.dim, n.window, "latent", 0), []).append(r)
     groups, group_of_run = [], {}
     for g, (key, runs) in enumerate(keyed.items()):
-        groups.append(GroupLayout(key[0], key[1], key[2], tuple(runs), key[3]))
+        groups.append(GroupLayout(key[0], key[1], key[2], tuple(runs), key[3], key[4]))
         for r in runs:
             group_of_run[r] = g
     return groups, group_of_run

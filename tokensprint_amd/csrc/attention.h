@@ -24,6 +24,8 @@ struct AttentionArgs {
   const float* slopes;    // [nq] or null: slope * (position - key) is taken off a score
   float temp_coef;        // the query at position p is multiplied by
   int temp_every;         // 1 + temp_coef ln(floor((p + 1) / temp_every) + 1); 0: by one
+  int keep;               // the sequence's first `keep` keys stay visible whatever window or
+                          // chunk says (causality aside); 0: none
 };
 
 // The first key the query at `pos` sees.
@@ -31,6 +33,22 @@ __device__ __forceinline__ int first_visible(const AttentionArgs& a, int pos) {
   int lo = (a.window > 0) ? max(0, pos - a.window + 1) : 0;
   if (a.chunk > 0) lo = max(lo, max(pos, 0) / a.chunk * a.chunk);
   return lo;
+}
+
+// The keys a tile of queries walks, as one stretch [origin, last position] of walk
+// coordinates: from `begin` on (the first visible key of the tile's first query, rounded
+// down to a block) a coordinate is the key's position; the kept first keys, in whole blocks,
+// stand right in front of `begin`, so the positions between them and the window are never
+// visited.  Without kept keys, or where they reach up to the window, nothing is left out.
+// ALIGN: keys in a block.
+struct KeyWalk {
+  int begin, origin;
+  __device__ __forceinline__ int real(int v) const { return v < begin ? v - origin : v; }
+};
+template <int ALIGN>
+__device__ __forceinline__ KeyWalk key_walk(const AttentionArgs& a, int first) {
+  const int begin = first & ~(ALIGN - 1);
+  return KeyWalk{begin, begin - min((a.keep + ALIGN - 1) & ~(ALIGN - 1), begin)};
 }
 
 // Whether scores are more than scale times the product: a cap, a distance bias or a

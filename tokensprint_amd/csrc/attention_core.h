@@ -64,25 +64,28 @@ struct PageCursor {
   ConstTable table;   // block table row of the entry
   int page_size;      // with PAGE16 a power of two >= 16
   int last_key;
+  KeyWalk walk;       // blocks are named by walk coordinates (attention.h)
   int next0, next1;   // page ids of the two 16-key blocks of the next call (two
                       // scalars: an array indexed at run time would live in memory)
   __device__ __forceinline__ int fetch(int k0) const {          // k0 is wave-uniform
     return k0 <= last_key ? table[k0 >> (__builtin_ctz(page_size))] : -1;
   }
-  __device__ __forceinline__ void start(int kb) {
+  __device__ __forceinline__ void start(int v) {
+    const int kb = walk.real(v);
     next0 = fetch(kb);
     next1 = fetch(kb + 16);
   }
 };
 
-// Loads the K and V operands of keys [kb, kb + 32).  With PAGE16 calls must come in
+// Loads the K and V operands of the 32 keys at walk coordinate `v`.  With PAGE16 calls must come in
 // steps of `stride` keys from the cursor's start (the cursor holds this call's pages and
-// then fetches those of kb + stride).
+// then fetches those of v + stride).
 template <int HD, bool PAGE16>
 __device__ __forceinline__ void load_kv_block(KvBlock<HD>& b, const AttentionArgs& a,
                                               const int* table, PageCursor& cur, int kvh,
-                                              int kb, int stride, int r, int g) {
+                                              int v, int stride, int r, int g) {
   constexpr int KS = KvBlock<HD>::KS, DB = KvBlock<HD>::DB;
+  const int kb = cur.walk.real(v);
   const bf16_t* kp = (const bf16_t*)a.k_pages;
   const bf16_t* vp = (const bf16_t*)a.v_pages;
   const int P = a.page_size;
@@ -133,7 +136,7 @@ __device__ __forceinline__ void load_kv_block(KvBlock<HD>& b, const AttentionArg
 #pragma unroll
   for (int db = 0; db < DB; ++db)
     b.v[db] = __builtin_shufflevector(vh[0][db], vh[1][db], 0, 1, 2, 3, 4, 5, 6, 7);
-  if (PAGE16) cur.start(kb + stride);
+  if (PAGE16) cur.start(v + stride);
 }
 
 // The same block with its keys assigned to the rows of the two score products so that lane
@@ -145,9 +148,10 @@ __device__ __forceinline__ void load_kv_block(KvBlock<HD>& b, const AttentionArg
 // `stride` keys from the cursor's start.
 template <int HD>
 __device__ __forceinline__ void load_kv_block_wide(KvBlock<HD>& b, const AttentionArgs& a,
-                                                   PageCursor& cur, int kvh, int kb, int stride,
+                                                   PageCursor& cur, int kvh, int v, int stride,
                                                    int r, int g) {
   constexpr int KS = KvBlock<HD>::KS, DB = KvBlock<HD>::DB;
+  const int kb = cur.walk.real(v);
   static_assert(HD % 32 == 0, "whole 32-element slices");
   const bf16_t* kp = (const bf16_t*)a.k_pages;
   const bf16_t* vp = (const bf16_t*)a.v_pages;
@@ -181,7 +185,7 @@ __device__ __forceinline__ void load_kv_block_wide(KvBlock<HD>& b, const Attenti
 #pragma unroll
     for (int db = 0; db < DB; ++db) b.v[db] = v_ok ? b.v[db] : zero8;
   }
-  cur.start(kb + stride);
+  cur.start(v + stride);
 }
 
 // One query tile's running state.
@@ -193,6 +197,7 @@ struct TileState {
   f32x4 o[DB];
   float m, l;         // l: this lane's share of the row's sum of weights (row_sum adds the four)
   int pos, lo;        // this lane's row: position and first visible key (pos = -1: no row)
+  int keep;           // keys below this are visible too
 };
 
 // The sum of weights of a lane's query row: the shares of the four lanes that hold the row.
@@ -263,7 +268,7 @@ __device__ __forceinline__ void tile_update(TileState<HD>& t, const KvBlock<HD>&
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
         const int key = PERM ? kb + g * 8 + blk * 4 + i : kb + blk * 16 + g * 4 + i;
-        st[blk][i] = (key <= t.pos && key >= t.lo) ? st[blk][i] : -INFINITY;
+        st[blk][i] = (key <= t.pos && (key >= t.lo || key < t.keep)) ? st[blk][i] : -INFINITY;
       }
   }
   const float mx = max2(max2(max2(max2(st[0][0], st[0][1]), st[0][2]),

@@ -214,7 +214,8 @@ __global__ __launch_bounds__(decode_waves<HD>() * kWave) void attention_decode_k
   const int last = new_key ? pos - 1 : pos;                   // last key walked from the cache
   const int lo = first_visible(a, pos);
   // chunks of this split: the arithmetic of attention_merge (from pos, not from last)
-  const int c_first = lo / kChunk, c_last = pos / kChunk;
+  const KeyWalk walk = key_walk<32>(a, lo);
+  const int c_first = walk.origin / kChunk, c_last = pos / kChunk;
   const int per = (c_last - c_first + ma.num_splits) / ma.num_splits;
   const int c0 = c_first + split * per, c1 = min(c0 + per, c_last + 1);
   if (c0 > c_last) {   // more splits than chunks: a neutral partial, no data touched
@@ -231,13 +232,14 @@ __global__ __launch_bounds__(decode_waves<HD>() * kWave) void attention_decode_k
   TileState<HD> t;
   t.pos = row_ok ? last : -1;
   t.lo = lo;
+  t.keep = a.keep;
   const float scale_log2 = a.scale * 1.44269504088896341f;
   ScoreExtra x;
   if (EXTRA) x = score_extra(a, head, row_ok ? pos : -1);   // distances from the query's own position
   const int stride = walkers * 32;
-  const int key_begin = max(c0 * kChunk, lo & ~31) + wave * 32;
+  const int key_begin = max(c0 * kChunk, walk.origin) + wave * 32;
   const int key_end = (prep_wave || key_wave) ? 0 : min(c1 * kChunk, last + 1);
-  PageCursor cur{(ConstTable)table, a.page_size, last, -1, -1};
+  PageCursor cur{(ConstTable)table, a.page_size, last, walk, -1, -1};
   KvBlock<HD> A, B;
   // head sizes in whole 32-element slices take the blocks with 16-byte value loads
   constexpr bool kWide = HD % 32 == 0;
@@ -317,14 +319,18 @@ __global__ __launch_bounds__(decode_waves<HD>() * kWave) void attention_decode_k
     load_query<HD>(t, (const bf16_t*)a.q + ((int64_t)token * a.nq + head) * HD, row_ok, g);
   }
 
-  for (int kb = key_begin; kb < key_end; kb += 2 * stride) {
-    if (kb + stride < key_end)
-      load_block(B, kb + stride);
-    tile_update<HD, false, kWide, EXTRA>(t, A, kb, scale_log2, kb + 31 <= last && kb >= lo, g, &x);
-    if (kb + stride >= key_end) break;
-    if (kb + 2 * stride < key_end)
-      load_block(A, kb + 2 * stride);
-    tile_update<HD, false, kWide, EXTRA>(t, B, kb + stride, scale_log2, kb + stride + 31 <= last && kb + stride >= lo, g, &x);
+  auto update = [&](const KvBlock<HD>& b, int v) {
+    const int kb = walk.real(v);
+    tile_update<HD, false, kWide, EXTRA>(t, b, kb, scale_log2, kb + 31 <= last && kb >= lo, g, &x);
+  };
+  for (int v = key_begin; v < key_end; v += 2 * stride) {
+    if (v + stride < key_end)
+      load_block(B, v + stride);
+    update(A, v);
+    if (v + stride >= key_end) break;
+    if (v + 2 * stride < key_end)
+      load_block(A, v + 2 * stride);
+    update(B, v + stride);
   }
   f32x4 (&o)[DB] = t.o;
   float m = t.m, l = row_sum<HD>(t);

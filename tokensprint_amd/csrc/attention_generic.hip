@@ -3,7 +3,8 @@
 // float32 path and of shapes the matrix-core kernels do not take.
 //
 // One workgroup of four wavefronts per (query token, query head).  Keys are cut into tiles
-// of 64 starting at the first visible key; wavefront w walks tiles w, w + 4, ... and the
+// of 64 starting at the first visible key (kept first keys, where there are any, right in
+// front of the window's); wavefront w walks tiles w, w + 4, ... and the
 // four partial results are merged in wavefront order, so the partition, and with it the
 // rounding, depends only on the token's position and the window, never on how the step was
 // cut or batched.  (A decode step of few requests has few such pairs: with a wavefront
@@ -53,9 +54,10 @@ __global__ __launch_bounds__(kWavesPerBlock* kWave) void attention_generic_kerne
 
   float m = -INFINITY, l = 0.f;
   float acc[kMaxHeadDim / kWave] = {};
-  for (int j0 = lo + wave * kWave; j0 <= pos; j0 += kWavesPerBlock * kWave) {
-    const int j = j0 + lane;
-    const bool valid = j <= pos;
+  const KeyWalk walk = key_walk<1>(a, lo);
+  for (int j0 = walk.origin + wave * kWave; j0 <= pos; j0 += kWavesPerBlock * kWave) {
+    const int j = walk.real(j0 + lane);
+    const bool valid = j0 + lane <= pos;
     float s = -INFINITY;
     int64_t row = -1;
     if (valid) {
@@ -93,7 +95,8 @@ __global__ __launch_bounds__(kWavesPerBlock* kWave) void attention_generic_kerne
       // the first visible key, which a window puts anywhere); in key order either way
       for (int jj = 0; jj < n; jj += 4) {
         const int64_t vrow = row_s[wave][jj];
-        const bool whole = jj + 3 < n && vrow >= 0 && ((j0 + jj) & 3) == 0;
+        const int j4 = walk.real(j0 + jj);
+        const bool whole = jj + 3 < n && vrow >= 0 && (j4 & 3) == 0 && walk.real(j0 + jj + 3) == j4 + 3;
         if (whole) {
 #pragma unroll
           for (int r = 0; r < kMaxHeadDim / kWave; ++r) {
@@ -173,6 +176,7 @@ int ts_check_attention_args(const AttentionArgs& a, const char* who) {
     TS_FAIL("%s: page_size=%d table_width=%d num_pages=%d", who, a.page_size, a.table_width,
             a.num_pages);
   if (a.window < 0) TS_FAIL("%s: window=%d", who, a.window);
+  if (a.keep < 0) TS_FAIL("%s: keep=%d", who, a.keep);
   if (a.chunk < 0 || a.softcap < 0.f || a.temp_every < 0)
     TS_FAIL("%s: chunk=%d softcap=%g temp_every=%d", who, a.chunk, a.softcap, a.temp_every);
   return 0;

@@ -55,8 +55,8 @@ __global__ __launch_bounds__(256) void attention_merge_kernel(AttentionMfmaArgs 
       for (int i = 0; i < DC; ++i) part[j][i] = args.partial_o[slot * HD + i * 16 + dc];
     }
     if (s0 == 0) {
-      const int lo_tile = first_visible(a, pos_first);
-      const int nchunks = pos_last / kChunk - lo_tile / kChunk + 1;
+      const int origin = key_walk<32>(a, first_visible(a, pos_first)).origin;
+      const int nchunks = pos_last / kChunk - origin / kChunk + 1;
       const int per = (nchunks - 1 + S) / S;
       used = min(S, (nchunks + per - 1) / per);
     }

@@ -39,8 +39,8 @@ __global__ __launch_bounds__(256, HD <= 128 ? 2 : 1) void attention_mfma_kernel(
   // key range of the tile and my share of its chunks
   const int pos_first = uniform(a.positions[tok0]);           // positions are consecutive
   const int pos_last = pos_first + ntok - 1;
-  const int lo_tile = first_visible(a, pos_first);
-  const int c_first = lo_tile / kChunk, c_last = pos_last / kChunk;
+  const KeyWalk walk = key_walk<32>(a, first_visible(a, pos_first));
+  const int c_first = walk.origin / kChunk, c_last = pos_last / kChunk;
   const int per = (c_last - c_first + args.num_splits) / args.num_splits;   // ceil(n / splits)
   const int c0 = c_first + split * per, c1 = min(c0 + per, c_last + 1);
   if (c0 > c_last) {   // more splits than chunks: a neutral partial, no data touched
@@ -55,6 +55,7 @@ __global__ __launch_bounds__(256, HD <= 128 ? 2 : 1) void attention_mfma_kernel(
   TileState<HD> t;
   t.pos = row_ok ? pos_first + ti : -1;
   t.lo = first_visible(a, t.pos);
+  t.keep = a.keep;
   load_query<HD>(t, (const bf16_t*)a.q + ((int64_t)token * a.nq + head) * HD, row_ok, g);
   const float scale_log2 = a.scale * 1.44269504088896341f;
   ScoreExtra x;
@@ -62,9 +63,9 @@ __global__ __launch_bounds__(256, HD <= 128 ? 2 : 1) void attention_mfma_kernel(
   const int lo_last = first_visible(a, pos_last);
 
   constexpr int kStride = COOP ? 128 : 32;
-  const int key_begin = max(c0 * kChunk, lo_tile & ~31) + (COOP ? wave * 32 : 0);
+  const int key_begin = max(c0 * kChunk, walk.origin) + (COOP ? wave * 32 : 0);
   const int key_end = min(c1 * kChunk, pos_last + 1);
-  PageCursor cur{(ConstTable)table, a.page_size, pos_last, -1, -1};
+  PageCursor cur{(ConstTable)table, a.page_size, pos_last, walk, -1, -1};
   if (PAGE16) cur.start(key_begin);
 
   KvBlock<HD> A, B;
@@ -76,13 +77,16 @@ __global__ __launch_bounds__(256, HD <= 128 ? 2 : 1) void attention_mfma_kernel(
     else load_kv_block<HD, PAGE16>(b, a, table, cur, kvh, kb, kStride, r, g);
   };
   if (key_begin < key_end) load_block(A, key_begin);
-  for (int kb = key_begin; kb < key_end; kb += 2 * kStride) {
-    if (kb + kStride < key_end) load_block(B, kb + kStride);
-    tile_update<HD, false, kWide, EXTRA>(t, A, kb, scale_log2, kb + 31 <= pos_first && kb >= lo_last, g, &x);
-    if (kb + kStride >= key_end) break;
-    if (kb + 2 * kStride < key_end) load_block(A, kb + 2 * kStride);
-    tile_update<HD, false, kWide, EXTRA>(t, B, kb + kStride, scale_log2,
-                                         kb + kStride + 31 <= pos_first && kb + kStride >= lo_last, g, &x);
+  auto update = [&](const KvBlock<HD>& b, int v) {
+    const int kb = walk.real(v);
+    tile_update<HD, false, kWide, EXTRA>(t, b, kb, scale_log2, kb + 31 <= pos_first && kb >= lo_last, g, &x);
+  };
+  for (int v = key_begin; v < key_end; v += 2 * kStride) {
+    if (v + kStride < key_end) load_block(B, v + kStride);
+    update(A, v);
+    if (v + kStride >= key_end) break;
+    if (v + 2 * kStride < key_end) load_block(A, v + 2 * kStride);
+    update(B, v + kStride);
   }
   f32x4 (&o)[DB] = t.o;
   float m = t.m, l = row_sum<HD>(t);

@@ -49,6 +49,7 @@ __global__ __launch_bounds__(256) void attention_prefill_kernel(AttentionMfmaArg
     const bool row_ok = ti < tq && t < ntok && hh < group;
     ts[j].pos = row_ok ? pos_first + t : -1;
     ts[j].lo = first_visible(a, ts[j].pos);
+    ts[j].keep = a.keep;
     tile_first[j] = pos_first + j * tq;
     tile_last[j] = j * tq < ntok ? pos_first + min(ntok, (j + 1) * tq) - 1 : -1;
     tile_lo[j] = first_visible(a, tile_first[j]);
@@ -57,14 +58,16 @@ __global__ __launch_bounds__(256) void attention_prefill_kernel(AttentionMfmaArg
                    ((int64_t)(tok0 + min(t, ntok - 1)) * a.nq + head) * HD, row_ok, g);
   }
 
-  const int key_begin = lo_all & ~31;
-  PageCursor cur{(ConstTable)table, a.page_size, pos_last, -1, -1};
+  const KeyWalk walk = key_walk<32>(a, lo_all);
+  const int key_begin = walk.origin;
+  PageCursor cur{(ConstTable)table, a.page_size, pos_last, walk, -1, -1};
   if (PAGE16) cur.start(key_begin);
 
-  auto work = [&](const KvBlock<HD>& b, int kb) {
+  auto work = [&](const KvBlock<HD>& b, int v) {
+    const int kb = walk.real(v);
 #pragma unroll
     for (int j = 0; j < TPW; ++j) {
-      if (kb > tile_last[j] || kb + 31 < tile_lo[j]) continue;        // scalar conditions
+      if (kb > tile_last[j] || (kb + 31 < tile_lo[j] && kb >= a.keep)) continue;   // scalar conditions
       const bool interior = kb + 31 <= tile_first[j] && kb >= tile_lo_last[j];
       tile_update<HD>(ts[j], b, kb, scale_log2, interior, g);
     }
@@ -212,6 +215,7 @@ __global__ __launch_bounds__(256 * H, H == 1 ? 3 : 2) void attention_prefill_asy
     TileState<HD> t;
     t.pos = row_ok ? pos_first + ti : -1;
     t.lo = first_visible(a, t.pos);
+    t.keep = a.keep;
     const int tile_first = pos_first + wave * tq;
     const int tile_last = wave * tq < ntok ? pos_first + min(ntok, (wave + 1) * tq) - 1 : -1;
     const int tile_lo = first_visible(a, tile_first);
@@ -222,17 +226,18 @@ __global__ __launch_bounds__(256 * H, H == 1 ? 3 : 2) void attention_prefill_asy
     // The item's blocks of 32 keys, numbered from its first; this set of waves takes
     // blocks set, set + H, ...: `mine` of them, numbered j here.  Every set makes the same
     // number of turns (a barrier each), the last of them idle for a set with one block less.
-    const int key_begin = lo_all & ~31;
+    const KeyWalk walk = key_walk<32>(a, lo_all);
+    const int key_begin = walk.origin;
     const int nblocks = ((pos_last - key_begin) >> 5) + 1;
     const int turns = (nblocks + H - 1) / H;
     const int mine = (nblocks - set + H - 1) / H;
     const int kb_first = key_begin + 32 * set;
-    PageCursor cur{(ConstTable)table, P, pos_last, -1, -1};
+    PageCursor cur{(ConstTable)table, P, pos_last, walk, -1, -1};
     cur.start(kb_first);
     // issue the loads of this set's block j into ring buffer `to`; calls come in order of
     // j, as the cursor needs
     auto issue = [&](int j, int to) {
-      const int kb = kb_first + 32 * H * j;
+      const int v = kb_first + 32 * H * j, kb = walk.real(v);
       const int in0 = kb & (P - 1), in1 = (kb + 16) & (P - 1);
       const int64_t p0 = (int64_t)max(cur.next0, 0) * page_stride, p1 = (int64_t)max(cur.next1, 0) * page_stride;
       const bf16_t* kb0 = k_head + p0 + in0 * HD;
@@ -246,13 +251,13 @@ __global__ __launch_bounds__(256 * H, H == 1 ? 3 : 2) void attention_prefill_asy
       for (int i = 0; i < KQ; ++i) lds_dma16(kbase + k_off[i], &kdst[wave + 4 * i][0]);
 #pragma unroll
       for (int i = 0; i < VQ; ++i) lds_dma16(vbase + v_off[i], &vdst[wave + 4 * i][0]);
-      cur.start(kb + 32 * H);
+      cur.start(v + 32 * H);
     };
 
     // One turn: block j is worked on out of ring buffer `from` while block j + 2 is sent
     // for into buffer `to`, which block j - 1 was read from.
     auto turn = [&](int j, int from, int to) {
-      const int kb = kb_first + 32 * H * j;
+      const int kb = walk.real(kb_first + 32 * H * j);
       // this wave's share of block j has arrived: at most block j + 1's loads are in flight
       if (j + 1 < mine) __builtin_amdgcn_s_waitcnt(0x0F70 | kLoads);
       else __builtin_amdgcn_s_waitcnt(0x0F70);
@@ -268,7 +273,7 @@ __global__ __launch_bounds__(256 * H, H == 1 ? 3 : 2) void attention_prefill_asy
       // others by a whole turn, and loads sent for before the barrier could land while a
       // slower wave still reads that buffer.
       if (j + 2 < mine) issue(j + 2, to);
-      if (j < mine && kb <= tile_last && kb + 31 >= tile_lo) {
+      if (j < mine && kb <= tile_last && (kb + 31 >= tile_lo || kb < a.keep)) {
         const Slots kcur = ring + from * kSlots, vcur = kcur + 2 * KS;
         KvBlock<HD> b;
 #pragma unroll
@@ -429,7 +434,7 @@ __device__ __forceinline__ void tile_update64(TileState<HD>& t, bf16x8 (*buf)[kW
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
         const int key = kb + (j / 2) * 32 + g * 8 + (j % 2) * 4 + i;
-        st[j][i] = (key <= t.pos && key >= t.lo) ? st[j][i] : -INFINITY;
+        st[j][i] = (key <= t.pos && (key >= t.lo || key < t.keep)) ? st[j][i] : -INFINITY;
       }
   }
   float mx = max2(max2(st[0][0], st[0][1]), max2(st[0][2], st[0][3]));
@@ -578,6 +583,7 @@ __device__ __forceinline__ void attention_prefill_wide(const AttentionMfmaArgs& 
     TileState<HD> t;
     t.pos = row_ok ? pos_first + ti : -1;
     t.lo = first_visible(a, t.pos);
+    t.keep = a.keep;
     ScoreExtra x;
     if (EXTRA) x = score_extra(a, head, t.pos);
     const int tile_first = pos_first + wave * tq;
@@ -602,7 +608,8 @@ __device__ __forceinline__ void attention_prefill_wide(const AttentionMfmaArgs& 
     // The item's turns of 64 keys, numbered from its first; this set takes turns set,
     // set + H, ...: `mine` of them, numbered j here.  Every set passes the same number of
     // barriers.
-    const int key_begin = lo_all & ~63;
+    const KeyWalk walk = key_walk<64>(a, lo_all);
+    const int key_begin = walk.origin;
     const int nturns = ((pos_last - key_begin) >> 6) + 1;
     const int rounds = (nturns + H - 1) / H;
     const int mine = (nturns - set + H - 1) / H;
@@ -614,7 +621,8 @@ __device__ __forceinline__ void attention_prefill_wide(const AttentionMfmaArgs& 
     // the scalar loads, so it is done where they are used, a turn later.
     int nx[4];
     typedef int Ids4 __attribute__((ext_vector_type(4), aligned(4)));
-    auto fetch_ids = [&](int kb) {
+    auto fetch_ids = [&](int v) {
+      const int kb = walk.real(v);
       const int i0 = kb >> lp;
       if (P16 && i0 + 3 <= last_page) {        // four consecutive pages: one scalar load
         const Ids4 ids = *(const Ids4 __attribute__((address_space(4)))*)(table + i0);
@@ -627,7 +635,7 @@ __device__ __forceinline__ void attention_prefill_wide(const AttentionMfmaArgs& 
     fetch_ids(kb_first);
 
     auto issue = [&](int j, int to) {
-      const int kb = kb_first + 64 * H * j;
+      const int v = kb_first + 64 * H * j, kb = walk.real(v);
       const Slots dst = ring + to * kBuf;
 #pragma unroll
       for (int sb = 0; sb < 2; ++sb) {
@@ -641,11 +649,11 @@ __device__ __forceinline__ void attention_prefill_wide(const AttentionMfmaArgs& 
           lds_dma16(src, &dst[sb * kSlots + wave + TILES * i][0]);
         }
       }
-      fetch_ids(kb + 64 * H);
+      fetch_ids(v + 64 * H);
     };
 
     auto turn = [&](int j, int from, int to) {
-      const int kb = kb_first + 64 * H * j;
+      const int kb = walk.real(kb_first + 64 * H * j);
       // this wave's share of turn j has arrived: at most the turn after it is in flight
       if (kAhead == 2 && j + 1 < mine) __builtin_amdgcn_s_waitcnt(0x0F70 | (2 * L));
       else __builtin_amdgcn_s_waitcnt(0x0F70);
@@ -656,7 +664,7 @@ __device__ __forceinline__ void attention_prefill_wide(const AttentionMfmaArgs& 
       // this one, after this turn's key operands have been asked for, so that LDS answers
       // meanwhile)
       auto send = [&]() { if (j + kAhead < mine) issue(j + kAhead, to); };
-      if (j < mine && kb <= tile_last && kb + 63 >= tile_lo)
+      if (j < mine && kb <= tile_last && (kb + 63 >= tile_lo || kb < a.keep))
         tile_update64<HD, true, EXTRA>(t, ring + from * kBuf, lane, kb, scale_log2,
                                        kb + 63 <= tile_first && kb >= tile_lo_last, g, send, &x);
       else

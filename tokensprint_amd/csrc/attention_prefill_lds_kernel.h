@@ -56,6 +56,7 @@ __global__ __launch_bounds__(256, HD <= 128 ? 4 : 1) void attention_prefill_lds_
   TileState<HD> t;
   t.pos = row_ok ? pos_first + ti : -1;
   t.lo = first_visible(a, t.pos);
+  t.keep = a.keep;
   ScoreExtra x;
   if (EXTRA) x = score_extra(a, head, t.pos);
   const int tile_first = pos_first + wave * tq;
@@ -69,8 +70,9 @@ __global__ __launch_bounds__(256, HD <= 128 ? 4 : 1) void attention_prefill_lds_
   const bf16_t* vp = (const bf16_t*)a.v_pages;
   const bf16x8 zero8 = {0, 0, 0, 0, 0, 0, 0, 0};
   const bf16x4 zero4 = {0, 0, 0, 0};
-  PageCursor cur{(ConstTable)table, P, pos_last, -1, -1};
-  const int key_begin = lo_all & ~31;
+  const KeyWalk walk = key_walk<32>(a, lo_all);
+  PageCursor cur{(ConstTable)table, P, pos_last, walk, -1, -1};
+  const int key_begin = walk.origin;
   cur.start(key_begin);
 
   // This wave's quarter of a block's operands: global -> registers.  The loads are
@@ -134,7 +136,8 @@ __global__ __launch_bounds__(256, HD <= 128 ? 4 : 1) void attention_prefill_lds_
     asm volatile("" : "+v"(off));
     return off;
   };
-  auto fetch = [&](Fetched& f, int kb) {
+  auto fetch = [&](Fetched& f, int v) {
+    const int kb = walk.real(v);
     const int in_page = kb & (P - 1);             // a block of 16 keys never straddles a page
     const int page0 = cur.next0, page1 = cur.next1;
     const bf16_t* kb0 = k_head + (int64_t)max(page0, 0) * k_page_stride + in_page * HD;
@@ -160,7 +163,7 @@ __global__ __launch_bounds__(256, HD <= 128 ? 4 : 1) void attention_prefill_lds_
         f.v[i] = *(const bf16x4*)((const char*)(v_blk[i] ? vb1 : vb0) + lane_offset(v_lane[i]));
       }
     }
-    cur.start(kb + 32);
+    cur.start(v + 32);
   };
   // registers -> LDS, operand layout.  (Blanking under a branch, taken only by the last
   // block of a context, was measured: slower than the selects it saves.)
@@ -200,10 +203,10 @@ __global__ __launch_bounds__(256, HD <= 128 ? 4 : 1) void attention_prefill_lds_
   for (int kb0 = key_begin; kb0 <= pos_last; kb0 += 32 * kAhead) {
 #pragma unroll
     for (int p = 0; p < kAhead; ++p) {
-      const int kb = kb0 + 32 * p;
-      if (kb > pos_last) break;
-      if (kb + 32 * kAhead <= pos_last) fetch(ring[p], kb + 32 * kAhead);
-      if (kb <= tile_last && kb + 31 >= tile_lo) {
+      const int v = kb0 + 32 * p, kb = walk.real(v);
+      if (v > pos_last) break;
+      if (v + 32 * kAhead <= pos_last) fetch(ring[p], v + 32 * kAhead);
+      if (kb <= tile_last && (kb + 31 >= tile_lo || kb < a.keep)) {
         KvBlock<HD> b;
 #pragma unroll
         for (int blk = 0; blk < 2; ++blk)
@@ -213,7 +216,7 @@ __global__ __launch_bounds__(256, HD <= 128 ? 4 : 1) void attention_prefill_lds_
         for (int db = 0; db < DB; ++db) b.v[db] = v_lds[buf][db][lane];
         tile_update<HD, true, false, EXTRA>(t, b, kb, scale_log2, kb + 31 <= tile_first && kb >= tile_lo_last, g, &x);
       }
-      if (kb + 32 <= pos_last) stash(ring[(p + 1) % kAhead], buf ^ 1);
+      if (v + 32 <= pos_last) stash(ring[(p + 1) % kAhead], buf ^ 1);
       __syncthreads();
       buf ^= 1;
     }

@@ -63,6 +63,19 @@ __device__ __forceinline__ float block_sum(float v, float* scratch) {
   return total;
 }
 
+// A gated feed-forward's unit, from the results of its two products (rounded to the
+// activation type first wherever a product makes it in its epilogue, as the path through
+// memory stores them): silu(gate) * up, or, with a
+// positive limit, g sigmoid(1.702 g) (u + 1) of g = min(gate, limit) and u = up held
+// between -limit and limit.
+__device__ __forceinline__ float gated_unit(float gate, float up, float limit) {
+  if (limit > 0.f) {
+    const float g = fminf(gate, limit), u = fminf(fmaxf(up, -limit), limit);
+    return g / (1.f + expf(-1.702f * g)) * (u + 1.f);
+  }
+  return gate / (1.f + expf(-gate)) * up;
+}
+
 // Dispatch a two-way element type code to a template argument.
 #define TS_DISPATCH_TYPE(code, T, ...)                    \
   if ((code) == TS_F32) { typedef float T; __VA_ARGS__; } \

@@ -506,10 +506,7 @@ __global__ __launch_bounds__(WK* kWave) void gemm_direct_kernel(DirectArgs a) {
     if (PAIR) {
 #pragma unroll
       for (int t = 0; t < 4; ++t) {
-        // the two products are rounded to the activation type first, as the unfused
-        // path stores them, then silu(gate) * up in float32
-        const float gt = (float)(bf16_t)v[t], up = (float)(bf16_t)(acc[1][mt][t] * rstd[mt]);
-        v[t] = gt / (1.f + expf(-gt)) * up;
+        v[t] = gated_unit((float)(bf16_t)v[t], (float)(bf16_t)(acc[1][mt][t] * rstd[mt]), a.limit);
       }
     }
     store4<TC>(C + (int64_t)m * N + n, v, N - n);

@@ -19,7 +19,7 @@ template <int MT, int WN, int WK, typename TC, bool PAIR>
 __global__ __launch_bounds__(WN* WK* kWave) void gemm_skinny_kernel(const bf16_t* __restrict__ A,
                                                           const bf16_t* __restrict__ W,
                                                           TC* __restrict__ C, int M, int N,
-                                                          int K) {
+                                                          int K, float limit) {
   constexpr int NW = PAIR ? 2 : 1;
   __shared__ f32x4 red[WK > 1 ? (WK - 1) * WN * NW * MT * kWave : 1];
   const int wave = threadIdx.x / kWave, lane = threadIdx.x % kWave;
@@ -105,10 +105,7 @@ __global__ __launch_bounds__(WN* WK* kWave) void gemm_skinny_kernel(const bf16_t
     if (PAIR) {
 #pragma unroll
       for (int t = 0; t < 4; ++t) {
-        // the two products are rounded to the activation type first, as the unfused
-        // path stores them, then silu(gate) * up in float32
-        const float gt = (float)(bf16_t)acc[0][mt][t], up = (float)(bf16_t)acc[1][mt][t];
-        v[t] = gt / (1.f + expf(-gt)) * up;
+        v[t] = gated_unit((float)(bf16_t)acc[0][mt][t], (float)(bf16_t)acc[1][mt][t], limit);
       }
     }
     store4<TC>(C + (int64_t)m * N + n, v, N - n);
@@ -136,6 +133,7 @@ struct StagedArgs {
   int kc;                   // K elements staged per round (multiple of WK*128, or >= K)
   int rstd_offset;          // byte offset in LDS of the fused form's row factors
   float eps;
+  float limit;              // PAIR: gated_unit's limit (0: silu)
 };
 
 template <int MT, int WN, int WK, typename TC, bool PAIR, bool NORM>
@@ -300,8 +298,7 @@ __global__ __launch_bounds__(WN* WK* kWave) void gemm_staged_kernel(StagedArgs a
     if (PAIR) {
 #pragma unroll
       for (int t = 0; t < 4; ++t) {
-        const float gt = (float)(bf16_t)v[t], up = (float)(bf16_t)(acc[1][mt][t] * rs);
-        v[t] = gt / (1.f + expf(-gt)) * up;
+        v[t] = gated_unit((float)(bf16_t)v[t], (float)(bf16_t)(acc[1][mt][t] * rs), a.limit);
       }
     }
     store4<TC>(C + (int64_t)m * N + n, v, N - n);
@@ -351,29 +348,30 @@ static int dispatch_staged(const StagedArgs& a, hipStream_t stream) {
 
 template <int MT, int WN, int WK, typename TC, bool PAIR>
 static void launch_skinny(const bf16_t* A, const bf16_t* W, TC* C, int M, int N, int K,
-                          hipStream_t stream) {
+                          float limit, hipStream_t stream) {
   dim3 grid((N + WN * 16 - 1) / (WN * 16), (M + MT * 16 - 1) / (MT * 16));
   hipLaunchKernelGGL((gemm_skinny_kernel<MT, WN, WK, TC, PAIR>), grid, dim3(WN * WK * kWave), 0,
-                     stream, A, W, C, M, N, K);
+                     stream, A, W, C, M, N, K, limit);
 }
 
 template <typename TC, bool PAIR>
 static int dispatch_skinny(const void* a, const void* w, void* c, int M, int N, int K,
-                           hipStream_t stream) {
+                           float limit, hipStream_t stream) {
   const bf16_t* A = (const bf16_t*)a;
   const bf16_t* W = (const bf16_t*)w;
   if (M <= 16) {   // few rows: both operands straight from global memory
-    launch_skinny<1, 4, 1, TC, PAIR>(A, W, (TC*)c, M, N, K, stream);
+    launch_skinny<1, 4, 1, TC, PAIR>(A, W, (TC*)c, M, N, K, limit, stream);
     return 0;
   }
   StagedArgs sa = {};
-  sa.A = A; sa.W = W; sa.C = c; sa.M = M; sa.N = N; sa.K = K;
+  sa.A = A; sa.W = W; sa.C = c; sa.M = M; sa.N = N; sa.K = K; sa.limit = limit;
   return dispatch_staged<TC, PAIR, false>(sa, stream);
 }
 
-// pair = 1: W is [2, N, K] (gate rows then up rows) and C[M, N] = silu(A Wg^T) * (A Wu^T).
+// pair = 1: W is [2, N, K] (gate rows then up rows) and C[M, N] = silu(A Wg^T) * (A Wu^T), or,
+// with a limit above 0, gated_unit's other form.
 extern "C" int ts_gemm_mfma_bf16(const void* a, const void* w, void* c, int c_type, int M,
-                                 int N, int K, int pair, hipStream_t stream) {
+                                 int N, int K, int pair, float limit, hipStream_t stream) {
   if (M <= 0 || N <= 0) return 0;
   if (K <= 0 || K % 8) TS_FAIL("gemm_mfma: K=%d must be a positive multiple of 8", K);
   if (((uintptr_t)a | (uintptr_t)w) & 15) TS_FAIL("gemm_mfma: operands must be 16-byte aligned");
@@ -382,14 +380,15 @@ extern "C" int ts_gemm_mfma_bf16(const void* a, const void* w, void* c, int c_ty
   if (!layout_wide(N, K)) {
     DirectArgs da = {};
     da.A = (const bf16_t*)a; da.W = (const bf16_t*)w; da.C = c; da.M = M; da.N = N; da.K = K;
+    da.limit = limit;
     rc = gemm_direct_launch(da, c_type, pair != 0, false, stream);
   } else if (pair) {
     if (c_type != TS_BF16) TS_FAIL("gemm_mfma: the paired product writes bfloat16");
-    rc = dispatch_skinny<bf16_t, true>(a, w, c, M, N, K, stream);
+    rc = dispatch_skinny<bf16_t, true>(a, w, c, M, N, K, limit, stream);
   } else if (c_type == TS_F32) {
-    rc = dispatch_skinny<float, false>(a, w, c, M, N, K, stream);
+    rc = dispatch_skinny<float, false>(a, w, c, M, N, K, limit, stream);
   } else if (c_type == TS_BF16) {
-    rc = dispatch_skinny<bf16_t, false>(a, w, c, M, N, K, stream);
+    rc = dispatch_skinny<bf16_t, false>(a, w, c, M, N, K, limit, stream);
   } else {
     TS_FAIL("gemm_mfma: unknown output type %d", c_type);
   }

@@ -58,6 +58,7 @@ struct TiledArgs {
   const float* norm_w;
   bf16_t* prepared;
   float* sumsq_out;
+  float limit;          // PAIR: gated_unit's limit (0: silu)
 };
 
 constexpr int kPlain = 0, kScaled = 1, kTail = 2;
@@ -379,6 +380,9 @@ __global__ __launch_bounds__(64 * GM * GN, 1) void gemm_tiled_kernel(TiledArgs g
     return;
   }
   TO* c = (TO*)g.c;
+  const bool clamped = PAIR && g.limit > 0.f;
+  const float top = clamped ? g.limit : INFINITY, lift = clamped ? 1.f : 0.f;
+  const float slope = clamped ? -1.702f * 1.44269504f : -1.44269504f;
   if constexpr (FORM == kScaled) {
     // (the barriers of the K loop lie between the factors' writes and these reads)
 #pragma unroll
@@ -407,7 +411,9 @@ __global__ __launch_bounds__(64 * GM * GN, 1) void gemm_tiled_kernel(TiledArgs g
           const float gv = (float)(TO)gate[e], uv = (float)(TO)up[e];
           // 64 values a lane at the very end of the kernel, the matrix cores idle: the
           // hardware's exp2 and reciprocal (an ulp each) instead of a division's ten steps
-          o[e] = gv * __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(gv * -1.44269504f)) * uv;
+          // (gated_unit's two forms: the clamps change nothing without a limit)
+          const float gc = fminf(gv, top), uc = fminf(fmaxf(uv, -top), top) + lift;
+          o[e] = gc * __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(gc * slope)) * uc;
         }
         store4<TO>(c + (int64_t)m * g.N + n, o, g.N - n);
       }

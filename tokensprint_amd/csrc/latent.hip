@@ -5,7 +5,8 @@
 //
 // Kernels: the preparation of a step's rows (norms of the two latents, rotation of the
 // shared key part, the write into the pages), the rotation of the queries' rotated part in
-// place, and attention.  (Carrying queries into the latent's space and results out of it
+// place, both of these in one kernel where queries and latent come out of one product, and
+// attention (with, where a layer has one, a sink per head in the softmax's denominator).  (Carrying queries into the latent's space and results out of it
 // are plain products over weights folded at load.)
 // Scores, softmax, rotation angles, norms: float32.  The rotation pairs dimension 2i with
 // 2i+1 and turns them by position * freq[i]; cosine and sine are computed here, at the
@@ -125,6 +126,88 @@ extern "C" int ts_rotate_interleaved(void* x, int type, const int* positions, co
   return 0;
 }
 
+// ---------------------------------------------------------------- rows of one product
+// x [T, ld] float32: the queries, heads x (kv_rank + rot_dim), then (`own`) the token's
+// latent (kv_rank) and shared key part (rot_dim).  The queries' rotated parts are turned in
+// place; the latent over its root mean square times kv_norm and the turned key part go to
+// the token's row of the pages.  One workgroup a token, which works out the position's
+// cosines and sines once.
+constexpr int kMaxRotPairs = 512;
+template <typename TC>
+__global__ __launch_bounds__(256) void latent_rows_kernel(
+    float* __restrict__ x, const float* __restrict__ kv_norm, const float* __restrict__ freqs,
+    TC* __restrict__ pages, const int* __restrict__ positions,
+    const int* __restrict__ entry_of_token, const int* __restrict__ table, int table_width,
+    int page_size, int ld, int heads, int own, int kv_rank, int rot_dim, int half, float eps) {
+  __shared__ float scratch[16], cos_s[kMaxRotPairs], sin_s[kMaxRotPairs];
+  const int t = blockIdx.x, dl = kv_rank + rot_dim;
+  float* row = x + (int64_t)t * ld;
+  const float* kv = row + heads * dl;
+  const int pos = positions[t];
+  for (int i = threadIdx.x; i < half; i += blockDim.x)
+    sincosf((float)pos * freqs[i], &sin_s[i], &cos_s[i]);
+  float rc = 0.f;
+  if (own) {
+    float ss = 0.f;
+    for (int i = threadIdx.x; i < kv_rank; i += blockDim.x) ss += kv[i] * kv[i];
+    rc = 1.0f / sqrtf(block_sum(ss, scratch) / (float)kv_rank + eps);
+  }
+  __syncthreads();
+  for (int idx = threadIdx.x; idx < heads * half; idx += blockDim.x) {
+    const int h = idx / half, i = idx % half;
+    float* v = row + h * dl + kv_rank + 2 * i;
+    const float a = v[0], b = v[1];
+    v[0] = a * cos_s[i] - b * sin_s[i];
+    v[1] = b * cos_s[i] + a * sin_s[i];
+  }
+  if (!own) return;
+  const int page = table[(int64_t)entry_of_token[t] * table_width + pos / page_size];
+  if (page < 0) return;     // an idle lane of a fixed-size batch: nothing to keep
+  TC* dst = pages + ((int64_t)page * page_size + pos % page_size) * dl;
+  for (int i = threadIdx.x; i < dl; i += blockDim.x) {
+    float v;
+    if (i < kv_rank) {
+      v = kv[i] * rc * kv_norm[i];
+    } else {
+      const int d = i - kv_rank;
+      v = kv[i];
+      if (d < 2 * half) {
+        const float o = kv[kv_rank + (d ^ 1)];
+        v = d & 1 ? v * cos_s[d / 2] + o * sin_s[d / 2] : v * cos_s[d / 2] - o * sin_s[d / 2];
+      }
+    }
+    dst[i] = from_f32<TC>(v);
+  }
+}
+
+extern "C" int ts_latent_rows(float* x, const float* kv_norm, const float* freqs, void* pages,
+                              int cache_type, const int* positions, const int* entry_of_token,
+                              const int* table, int table_width, int page_size, int num_tokens,
+                              int ld, int heads, int own, int kv_rank, int rot_dim, int rot_dims,
+                              float eps, hipStream_t stream) {
+  if (num_tokens <= 0) return 0;
+  const int dl = kv_rank + rot_dim;
+  if (heads <= 0 || kv_rank <= 0 || rot_dim < 0 || rot_dims < 0 || rot_dims % 2 ||
+      rot_dims > rot_dim || rot_dims / 2 > kMaxRotPairs || page_size <= 0 || table_width <= 0)
+    TS_FAIL("latent_rows: bad sizes heads=%d kv_rank=%d rot_dim=%d rot_dims=%d (at most %d turned)",
+            heads, kv_rank, rot_dim, rot_dims, 2 * kMaxRotPairs);
+  if (ld != heads * dl + (own ? dl : 0)) TS_FAIL("latent_rows: rows of %d", ld);
+  if (own && !kv_norm) TS_FAIL("latent_rows: no norm weight");
+  TS_DISPATCH_TYPE(cache_type, TC,
+      hipLaunchKernelGGL(latent_rows_kernel<TC>, dim3(num_tokens), dim3(256), 0, stream, x,
+                         kv_norm, freqs, (TC*)pages, positions, entry_of_token, table,
+                         table_width, page_size, ld, heads, own, kv_rank, rot_dim, rot_dims / 2,
+                         eps));
+  TS_CHECK_LAUNCH("latent_rows");
+  return 0;
+}
+
+// A head's sink in units of the softmax's weights relative to `m`; cut off where the output
+// has long become zero, so nothing overflows.
+__device__ __forceinline__ float sink_weight(float sink, float m) {
+  return expf(fminf(sink - m, 69.f));
+}
+
 // ---------------------------------------------------------------- attention
 // One wavefront per (token, head), four heads of a token to a workgroup (they read the same
 // rows).  Keys are cut into tiles of 64 starting at the first visible key, so the partition
@@ -140,7 +223,7 @@ __global__ __launch_bounds__(kLatentWaves* kWave) void latent_attention_kernel(
     const float* __restrict__ qa, const TC* __restrict__ pages, TO* __restrict__ out,
     const int* __restrict__ positions, const int* __restrict__ entry_of_token,
     const int* __restrict__ table, int table_width, int page_size, int heads, int kv_rank,
-    int rot_dim, int window, float scale) {
+    int rot_dim, int window, float scale, int q_ld, const float* __restrict__ sink) {
   extern __shared__ float lds[];      // per wave: q [dl], p [64], row numbers [64]
   const int wave = threadIdx.x / kWave, lane = threadIdx.x % kWave;
   const int dl = kv_rank + rot_dim;
@@ -154,7 +237,7 @@ __global__ __launch_bounds__(kLatentWaves* kWave) void latent_attention_kernel(
   const int pos = positions[t];
   const int lo = window > 0 ? max(0, pos - window + 1) : 0;
   const int* tab = table + (int64_t)entry_of_token[t] * table_width;
-  const float* q = qa + ((int64_t)t * heads + h) * dl;
+  const float* q = qa + (int64_t)t * q_ld + h * dl;
   for (int d = lane; d < dl; d += kWave) q_s[d] = q[d];
   __builtin_amdgcn_wave_barrier();
   const bool by4 = dl % 4 == 0 && ((uintptr_t)pages & 15) == 0;
@@ -206,6 +289,7 @@ __global__ __launch_bounds__(kLatentWaves* kWave) void latent_attention_kernel(
     }
     __builtin_amdgcn_wave_barrier();
   }
+  if (sink) l += sink_weight(sink[h], m);
   TO* o = out + ((int64_t)t * heads + h) * kv_rank;
   const float inv = l > 0.f ? 1.0f / l : 0.f;
 #pragma unroll
@@ -219,9 +303,11 @@ extern "C" int ts_latent_attention(const float* qa, const void* pages, int cache
                                    int out_type, const int* positions, const int* entry_of_token,
                                    const int* table, int table_width, int page_size,
                                    int num_tokens, int heads, int kv_rank, int rot_dim,
-                                   int window, float scale, hipStream_t stream) {
+                                   int window, float scale, int q_ld, const float* sink,
+                                   hipStream_t stream) {
   if (num_tokens <= 0) return 0;
   const int dl = kv_rank + rot_dim;
+  if (q_ld < heads * dl) TS_FAIL("latent_attention: query rows of %d", q_ld);
   if (heads <= 0 || kv_rank <= 0 || rot_dim < 0 || page_size <= 0 || table_width <= 0)
     TS_FAIL("latent_attention: bad sizes heads=%d kv_rank=%d rot_dim=%d", heads, kv_rank, rot_dim);
   if (kv_rank > kMaxRankPerLane * kWave || dl > kMaxLatent)
@@ -232,7 +318,8 @@ extern "C" int ts_latent_attention(const float* qa, const void* pages, int cache
   TS_DISPATCH_TYPE(cache_type, TC, TS_DISPATCH_TYPE(out_type, TO,
       hipLaunchKernelGGL((latent_attention_kernel<TC, TO>), grid, dim3(kLatentWaves * kWave), lds,
                          stream, qa, (const TC*)pages, (TO*)out, positions, entry_of_token, table,
-                         table_width, page_size, heads, kv_rank, rot_dim, window, scale)));
+                         table_width, page_size, heads, kv_rank, rot_dim, window, scale, q_ld,
+                         sink)));
   TS_CHECK_LAUNCH("latent_attention");
   return 0;
 }
@@ -255,7 +342,8 @@ extern "C" int ts_latent_attention(const float* qa, const void* pages, int cache
 typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8_l;
 
 struct LatentMfmaArgs {
-  const float* qa;          // [rows, dl], rows = tokens * heads
+  const float* qa;          // [tokens, q_ld]: the heads' rows of dl side by side (and, where
+                            // q_ld is larger, something else behind them)
   const bf16_t* pages;      // [pages, page_size, dl]
   void* out;                // [rows, kv_rank]
   const int* tiles;         // [num_tiles, 3]: first row, rows (1..16), entry
@@ -265,6 +353,8 @@ struct LatentMfmaArgs {
   float* part_ml;           // [num_tiles, splits, 16, 2]
   int table_width, page_size, heads, kv_rank, rot_dim, window, keys_per_split, splits;
   float scale;
+  int q_ld;
+  const float* sink;        // [heads] or null: a score that joins a row's denominator once
 };
 
 constexpr int kLatentPad = 8;     // elements between staged rows: operand reads spread over banks
@@ -303,7 +393,8 @@ __global__ __launch_bounds__(4 * kWave) void latent_attention_mfma_kernel(Latent
   const int k_end = min(k_begin + a.keys_per_split, hi_t + 1);
 
   bf16x8_l q[KS];
-  const float* qr = a.qa + (int64_t)my_row * dl;
+  const int my_head = my_row % a.heads;
+  const float* qr = a.qa + (int64_t)(my_row / a.heads) * a.q_ld + my_head * dl;
 #pragma unroll
   for (int s = 0; s < KS; ++s) {
     const int d0 = 32 * s + 8 * g;
@@ -395,6 +486,7 @@ __global__ __launch_bounds__(4 * kWave) void latent_attention_mfma_kernel(Latent
   }
   if (a.splits == 1) {
     if (!row_ok) return;
+    if (a.sink) l += sink_weight(a.sink[my_head], m);
     const float inv = l > 0.f ? 1.0f / l : 0.f;
     TO* orow = (TO*)a.out + (int64_t)my_row * a.kv_rank;
 #pragma unroll
@@ -444,6 +536,7 @@ __global__ __launch_bounds__(128) void latent_attention_merge_kernel(LatentMfmaA
       total += a.part_ml[2 * (base + 16 * s) + 1] * w;
     }
     total = wave_sum(total);
+    if (a.sink) total += sink_weight(a.sink[(a.tiles[3 * tile] + r) % a.heads], mx);
     if (threadIdx.x == 0) w_s[a.splits] = total > 0.f ? 1.0f / total : 0.f;
   }
   __syncthreads();
@@ -492,8 +585,10 @@ extern "C" int ts_latent_attention_mfma(const float* qa, const void* pages, void
                                         const int* positions, const int* table, int table_width,
                                         int page_size, int heads, int kv_rank, int rot_dim,
                                         int window, float scale, int keys_per_split, int splits,
-                                        float* part_o, float* part_ml, hipStream_t stream) {
+                                        float* part_o, float* part_ml, int q_ld,
+                                        const float* sink, hipStream_t stream) {
   if (num_tiles <= 0) return 0;
+  if (q_ld < heads * (kv_rank + rot_dim)) TS_FAIL("latent_attention_mfma: query rows of %d", q_ld);
   if (!ts_latent_attention_mfma_fits(kv_rank, rot_dim) || heads <= 0 || page_size <= 0)
     TS_FAIL("latent_attention_mfma: sizes kv_rank=%d rot_dim=%d are not served", kv_rank, rot_dim);
   if (splits < 1 || keys_per_split < 32 || keys_per_split % 32)
@@ -504,7 +599,7 @@ extern "C" int ts_latent_attention_mfma(const float* qa, const void* pages, void
   if (((uintptr_t)pages & 15) != 0) TS_FAIL("latent_attention_mfma: pages must start on 16 bytes");
   LatentMfmaArgs a{qa, (const bf16_t*)pages, out, tiles, positions, table, part_o, part_ml,
                    table_width, page_size, heads, kv_rank, rot_dim, window, keys_per_split, splits,
-                   scale};
+                   scale, q_ld, sink};
   const int dl = kv_rank + rot_dim;
   int rc;
   if (dl <= 96 && kv_rank <= 64) rc = launch_latent_mfma<3, 4>(a, num_tiles, waves, out_type, stream);

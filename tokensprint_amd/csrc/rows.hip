@@ -222,21 +222,21 @@ extern "C" int ts_add_rmsnorm(float* resid, const void* delta, int delta_type, c
 // gate_up is [rows, 2*inner]: gate in the first half of a row, up in the second.
 template <typename T>
 __global__ void silu_mul_kernel(const T* __restrict__ gu, T* __restrict__ out, int64_t total,
-                                int inner) {
+                                int inner, float limit) {
   for (int64_t i = blockIdx.x * (int64_t)blockDim.x + threadIdx.x; i < total;
        i += (int64_t)gridDim.x * blockDim.x) {
     const int64_t r = i / inner;
     const int c = (int)(i - r * inner);
     const float g = to_f32(gu[r * 2 * inner + c]);
     const float u = to_f32(gu[r * 2 * inner + inner + c]);
-    out[i] = from_f32<T>(g / (1.f + expf(-g)) * u);
+    out[i] = from_f32<T>(gated_unit(g, u, limit));
   }
 }
 
 // Eight bfloat16 per thread (inner a multiple of 8): 16-byte loads and stores.
 typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8_rows;
 __global__ void silu_mul_bf16x8_kernel(const bf16_t* __restrict__ gu, bf16_t* __restrict__ out,
-                                       int64_t units, int units_per_row) {
+                                       int64_t units, int units_per_row, float limit) {
   for (int64_t i = blockIdx.x * (int64_t)blockDim.x + threadIdx.x; i < units;
        i += (int64_t)gridDim.x * blockDim.x) {
     const int64_t r = i / units_per_row;
@@ -246,22 +246,19 @@ __global__ void silu_mul_bf16x8_kernel(const bf16_t* __restrict__ gu, bf16_t* __
     const bf16x8_rows u = *(const bf16x8_rows*)(gu + r * 2 * inner + inner + c);
     bf16x8_rows o;
 #pragma unroll
-    for (int j = 0; j < 8; ++j) {
-      const float gf = (float)g[j];
-      o[j] = (bf16_t)(gf / (1.f + expf(-gf)) * (float)u[j]);
-    }
+    for (int j = 0; j < 8; ++j) o[j] = (bf16_t)gated_unit((float)g[j], (float)u[j], limit);
     *(bf16x8_rows*)(out + r * inner + c) = o;
   }
 }
 
 extern "C" int ts_silu_mul(const void* gate_up, void* out, int type, int rows, int inner,
-                           hipStream_t stream) {
+                           float limit, hipStream_t stream) {
   if (rows <= 0) return 0;
   if (type == TS_BF16 && inner % 8 == 0 && (((uintptr_t)gate_up | (uintptr_t)out) & 15) == 0) {
     const int64_t units = (int64_t)rows * (inner / 8);
     const int blocks = (int)((units + 255) / 256 > 16384 ? 16384 : (units + 255) / 256);
     hipLaunchKernelGGL(silu_mul_bf16x8_kernel, dim3(blocks), dim3(256), 0, stream,
-                       (const bf16_t*)gate_up, (bf16_t*)out, units, inner / 8);
+                       (const bf16_t*)gate_up, (bf16_t*)out, units, inner / 8, limit);
     TS_CHECK_LAUNCH("silu_mul");
     return 0;
   }
@@ -269,7 +266,7 @@ extern "C" int ts_silu_mul(const void* gate_up, void* out, int type, int rows, i
   const int blocks = (int)((total + 255) / 256 > 65535 ? 65535 : (total + 255) / 256);
   TS_DISPATCH_TYPE(type, T,
                    hipLaunchKernelGGL(silu_mul_kernel<T>, dim3(blocks), dim3(256), 0, stream,
-                                      (const T*)gate_up, (T*)out, total, inner));
+                                      (const T*)gate_up, (T*)out, total, inner, limit));
   TS_CHECK_LAUNCH("silu_mul");
   return 0;
 }

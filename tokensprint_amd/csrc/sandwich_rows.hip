@@ -1,7 +1,9 @@
 // Row-wise kernels of layers that norm a sub-layer's output before adding it to the
 // residual stream, and of what such models put in front of the stream: a bigram-hashed
-// embedding with its norm, the add of a normalised output (alone, or with the next
-// sub-layer's norm), the norm with a token shift behind it, and the PolyNorm activation.
+// embedding with its norm, the add of a normalised output (alone, with the next
+// sub-layer's norm, or with the new stream's rows for a sub-layer that reads it as it is),
+// the gate of a token's own input to a layer, the norm with a token shift behind it, and the
+// PolyNorm activation.
 // One workgroup per row; every sum, root and product in float32.
 //
 // Per-request state (the previous token, the previous row of a token shift) lives in
@@ -91,27 +93,35 @@ extern "C" int ts_bigram_embed(const void* table, const void* bigram, int table_
 }
 
 // ---------------------------------------------------------------- add of a normalised output
-// resid += delta / rms(delta) * post_w; with NORM also out = resid / rms(resid) * norm_w.
-template <typename TO, bool NORM>
+// resid += delta / rms(delta) * post_w; then, by THEN, nothing more, or also
+// out = resid / rms(resid) * norm_w, or out = resid itself (rounded to out's type, for a
+// sub-layer that reads the stream as it is).
+constexpr int kThenNothing = 0, kThenNorm = 1, kThenRows = 2;
+
+template <typename TD, typename TO, int THEN>
 __global__ __launch_bounds__(1024) void postnorm_add_kernel(
-    float* __restrict__ resid, const float* __restrict__ delta, const float* __restrict__ post_w,
+    float* __restrict__ resid, const TD* __restrict__ delta, const float* __restrict__ post_w,
     const float* __restrict__ norm_w, TO* __restrict__ out, int width, float post_eps,
     float norm_eps) {
   __shared__ float scratch[16];
   const int64_t row = blockIdx.x;
   const int nt = blockDim.x;
   float* x = resid + row * width;
-  const float* d = delta + row * width;
+  const TD* d = delta + row * width;
+  TO* o = out + row * width;
   float dc[kRowItems], xc[kRowItems];
   float ss = 0.f;
 #pragma unroll
   for (int k = 0; k < kRowItems; ++k) {
     const int i = threadIdx.x + k * nt;
-    dc[k] = i < width ? d[i] : 0.f;
+    dc[k] = i < width ? to_f32(d[i]) : 0.f;
     xc[k] = i < width ? x[i] : 0.f;
     ss += dc[k] * dc[k];
   }
-  for (int i = threadIdx.x + kRowItems * nt; i < width; i += nt) ss += d[i] * d[i];
+  for (int i = threadIdx.x + kRowItems * nt; i < width; i += nt) {
+    const float v = to_f32(d[i]);
+    ss += v * v;
+  }
   const float r = inv_rms(block_sum(ss, scratch), width, post_eps);
   float ss2 = 0.f;
 #pragma unroll
@@ -120,17 +130,18 @@ __global__ __launch_bounds__(1024) void postnorm_add_kernel(
     if (i < width) {
       xc[k] = xc[k] + dc[k] * r * post_w[i];
       x[i] = xc[k];
+      if (THEN == kThenRows) o[i] = from_f32<TO>(xc[k]);
       ss2 += xc[k] * xc[k];
     }
   }
   for (int i = threadIdx.x + kRowItems * nt; i < width; i += nt) {
-    const float v = x[i] + d[i] * r * post_w[i];
+    const float v = x[i] + to_f32(d[i]) * r * post_w[i];
     x[i] = v;
+    if (THEN == kThenRows) o[i] = from_f32<TO>(v);
     ss2 += v * v;
   }
-  if (NORM) {
+  if (THEN == kThenNorm) {
     const float r2 = inv_rms(block_sum(ss2, scratch), width, norm_eps);
-    TO* o = out + row * width;
 #pragma unroll
     for (int k = 0; k < kRowItems; ++k) {
       const int i = threadIdx.x + k * nt;
@@ -142,21 +153,65 @@ __global__ __launch_bounds__(1024) void postnorm_add_kernel(
   }
 }
 
-extern "C" int ts_postnorm_add(float* resid, const float* delta, const float* post_w,
-                               float post_eps, const float* norm_w, float norm_eps, void* out,
-                               int out_type, int rows, int width, hipStream_t stream) {
+// With `norm_w` the norm of the new stream goes to `out`; with `out` alone the new stream.
+extern "C" int ts_postnorm_add(float* resid, const void* delta, int delta_type,
+                               const float* post_w, float post_eps, const float* norm_w,
+                               float norm_eps, void* out, int out_type, int rows, int width,
+                               hipStream_t stream) {
   if (rows <= 0) return 0;
   if (width <= 0) TS_FAIL("postnorm_add: bad width %d", width);
-  if (norm_w == nullptr) {
-    hipLaunchKernelGGL((postnorm_add_kernel<float, false>), dim3(rows), dim3(row_threads(width)),
-                       0, stream, resid, delta, post_w, nullptr, nullptr, width, post_eps, 0.f);
-  } else {
-    TS_DISPATCH_TYPE(out_type, TO,
-                     hipLaunchKernelGGL((postnorm_add_kernel<TO, true>), dim3(rows),
-                                        dim3(row_threads(width)), 0, stream, resid, delta, post_w,
-                                        norm_w, (TO*)out, width, post_eps, norm_eps));
-  }
+  if (norm_w && !out) TS_FAIL("postnorm_add: a norm without an output");
+  const dim3 grid(rows), block(row_threads(width));
+  TS_DISPATCH_TYPE(delta_type, TD, {
+    if (!out) {
+      hipLaunchKernelGGL((postnorm_add_kernel<TD, float, kThenNothing>), grid, block, 0, stream,
+                         resid, (const TD*)delta, post_w, nullptr, nullptr, width, post_eps, 0.f);
+    } else if (norm_w) {
+      TS_DISPATCH_TYPE(out_type, TO,
+                       hipLaunchKernelGGL((postnorm_add_kernel<TD, TO, kThenNorm>), grid, block, 0,
+                                          stream, resid, (const TD*)delta, post_w, norm_w,
+                                          (TO*)out, width, post_eps, norm_eps));
+    } else {
+      TS_DISPATCH_TYPE(out_type, TO,
+                       hipLaunchKernelGGL((postnorm_add_kernel<TD, TO, kThenRows>), grid, block, 0,
+                                          stream, resid, (const TD*)delta, post_w, nullptr,
+                                          (TO*)out, width, post_eps, 0.f));
+    }
+  });
   TS_CHECK_LAUNCH("postnorm_add");
+  return 0;
+}
+
+// ---------------------------------------------------------------- a token's own input
+// out[t, j] = gelu_tanh(z[t, j]) * table[ids[t], col + j], j < dim: the gate of what a
+// token's row of a table brings into a layer.  z float32 [T, dim], table [V, ld].
+__device__ __forceinline__ float gelu_tanh(float z) {
+  return 0.5f * z * (1.0f + tanhf(0.79788456080286536f * (z + 0.044715f * z * z * z)));
+}
+
+template <typename TW, typename TO>
+__global__ __launch_bounds__(256) void token_gate_kernel(
+    const float* __restrict__ z, const TW* __restrict__ table, const int* __restrict__ ids,
+    TO* __restrict__ out, int64_t total, int dim, int ld, int col) {
+  const int64_t idx = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
+  if (idx >= total) return;
+  const int64_t t = idx / dim;
+  const int j = (int)(idx - t * dim);
+  out[idx] = from_f32<TO>(gelu_tanh(z[idx]) * to_f32(table[(int64_t)ids[t] * ld + col + j]));
+}
+
+extern "C" int ts_token_gate(const float* z, const void* table, int table_type, const int* ids,
+                             void* out, int out_type, int num_tokens, int dim, int ld, int col,
+                             hipStream_t stream) {
+  if (num_tokens <= 0) return 0;
+  if (dim <= 0 || col < 0 || col + dim > ld)
+    TS_FAIL("token_gate: columns [%d, %d) of rows of %d", col, col + dim, ld);
+  const int64_t total = (int64_t)num_tokens * dim;
+  TS_DISPATCH_TYPE(table_type, TW, TS_DISPATCH_TYPE(out_type, TO,
+      hipLaunchKernelGGL((token_gate_kernel<TW, TO>), dim3((unsigned)((total + 255) / 256)),
+                         dim3(256), 0, stream, z, (const TW*)table, ids, (TO*)out, total, dim, ld,
+                         col)));
+  TS_CHECK_LAUNCH("token_gate");
   return 0;
 }
 

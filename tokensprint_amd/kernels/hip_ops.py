@@ -50,7 +50,7 @@ class AttentionArgs(Structure):
         ("nkv", c_int), ("hd", c_int), ("page_size", c_int), ("num_pages", c_int),
         ("window", c_int), ("scale", c_float), ("sink", c_void_p),
         ("chunk", c_int), ("softcap", c_float), ("slopes", c_void_p), ("temp_coef", c_float),
-        ("temp_every", c_int),
+        ("temp_every", c_int), ("keep", c_int),
     ]
 
 
@@ -286,15 +286,26 @@ class HipOps:
                    resid.shape[1], c_float(eps), self._stream())
         return out
 
-    def silu_mul(self, gate_up):
+    def silu_mul(self, gate_up, limit=None):
+        """gate_up [rows, gate | up] -> silu(gate) * up; with a `limit`, g sigmoid(1.702 g)
+        (u + 1) of g = min(gate, limit) and u = up held between -limit and limit."""
         self._check("gate_up", gate_up, self._FLOATS, ndim=2)
         rows, two_inner = gate_up.shape
         if two_inner % 2:
             raise ValueError("gate_up needs an even row width (gate half, up half)")
         out = torch.empty(rows, two_inner // 2, dtype=gate_up.dtype, device=self.device)
         self._call(self.lib.ts_silu_mul, _ptr(gate_up), _ptr(out), _TYPE_CODE[gate_up.dtype],
-                   rows, two_inner // 2, self._stream())
+                   rows, two_inner // 2, self._limit(limit), self._stream())
         return out
+
+    @staticmethod
+    def _limit(limit):
+        """A gated unit's limit as the kernels take it (0: there is none)."""
+        if limit is None:
+            return c_float(0.0)
+        if not limit > 0:
+            raise ValueError(f"a gated unit's limit must be positive, got {limit}")
+        return c_float(limit)
 
     # ------------------------------------------------------------ matrix product
     def linear(self, x, weight, out_dtype):
@@ -323,7 +334,7 @@ class HipOps:
         out = torch.empty(M, N, dtype=out_dtype, device=self.device)
         if self._mfma_ok(x, weight):
             self._call(self.lib.ts_gemm_mfma_bf16, _ptr(x), _ptr(weight), _ptr(out),
-                       _TYPE_CODE[out_dtype], M, N, K, 0, self._stream())
+                       _TYPE_CODE[out_dtype], M, N, K, 0, c_float(0.0), self._stream())
         else:
             self._call(self.lib.ts_gemm_fma, _ptr(x), _TYPE_CODE[x.dtype], _ptr(weight),
                        _TYPE_CODE[weight.dtype], _ptr(out), _TYPE_CODE[out_dtype], M, N, K,
@@ -341,9 +352,10 @@ class HipOps:
         self.lib.ts_gemm_library_candidates(8 if on else 1)
         return before
 
-    def gemm_tiled(self, x, weight, out_dtype, pair=False, tile=0):
+    def gemm_tiled(self, x, weight, out_dtype, pair=False, tile=0, limit=None):
         """The LDS-tiled product for many rows: x [M, K] bfloat16, weight [N, K] bfloat16
-        (with `pair` [2 N, K], gate rows then up rows, and the result is silu(gate) * up).
+        (with `pair` [2 N, K], gate rows then up rows, and the result is silu(gate) * up, or
+        with a `limit` silu_mul's other form).
         `tile` 0 lets the sizes choose the tile; another names one (the result is the same
         to the bit)."""
         self._check("x", x, torch.bfloat16, ndim=2)
@@ -354,7 +366,8 @@ class HipOps:
             raise ValueError(f"gemm_tiled: x {tuple(x.shape)}, weight {tuple(weight.shape)}")
         out = torch.empty(M, N, dtype=out_dtype, device=self.device)
         self._call(self.lib.ts_gemm_tiled_bf16, _ptr(x), _ptr(weight), _ptr(out),
-                   _TYPE_CODE[out_dtype], M, N, K, int(pair), tile, self._stream())
+                   _TYPE_CODE[out_dtype], M, N, K, int(pair), tile, self._limit(limit),
+                   self._stream())
         return out
 
     # Which rows and sizes go to the vendor library, to the LDS-tiled kernel or stay with
@@ -583,8 +596,9 @@ class HipOps:
                    int(silu_mul), self._stream())
         return out, resid_out
 
-    def linear_silu_mul(self, x, weight, out_dtype):
-        """silu(x Wg^T) * (x Wu^T) for weight = [Wg; Wu] stacked by rows -> [M, N/2]."""
+    def linear_silu_mul(self, x, weight, out_dtype, limit=None):
+        """silu(x Wg^T) * (x Wu^T) for weight = [Wg; Wu] stacked by rows -> [M, N/2]; with a
+        `limit` the gated unit is silu_mul's other form."""
         x = self._rows(x)
         self._check("x", x, self._FLOATS, ndim=2)
         self._check("weight", weight, self._FLOATS, ndim=2)
@@ -593,14 +607,14 @@ class HipOps:
             raise ValueError(f"linear_silu_mul: x {tuple(x.shape)}, weight {tuple(weight.shape)}")
         inner = weight.shape[0] // 2
         if self._tiled_pair_ok(x, weight, out_dtype):
-            return self.gemm_tiled(x, weight, out_dtype, pair=True)
+            return self.gemm_tiled(x, weight, out_dtype, pair=True, limit=limit)
         if (self._mfma_ok(x, weight) and out_dtype == torch.bfloat16
                 and not self._library_ok(x, weight, out_dtype)):
             out = torch.empty(M, inner, dtype=out_dtype, device=self.device)
             self._call(self.lib.ts_gemm_mfma_bf16, _ptr(x), _ptr(weight), _ptr(out),
-                       _TYPE_CODE[out_dtype], M, inner, K, 1, self._stream())
+                       _TYPE_CODE[out_dtype], M, inner, K, 1, self._limit(limit), self._stream())
             return out
-        return self.silu_mul(self.linear(x, weight, out_dtype))
+        return self.silu_mul(self.linear(x, weight, out_dtype), limit)
 
     # ------------------------------------------------------------ q/k preparation
     def _qk_args(self, qkv, batch, *, num_heads, kv_in_row, head_dim, q_weight, k_weight, eps,
@@ -719,10 +733,11 @@ class HipOps:
     # ------------------------------------------------------------ attention
     def paged_attention(self, q, batch, table, cache, *, num_heads, num_kv_heads, head_dim,
                         scale, window, sink=None, chunk=None, softcap=None, slopes=None,
-                        q_temp=None):
+                        q_temp=None, keep_first=0):
         """`sink`: float32 [num_heads] or None: a score per query head that joins the
         softmax's denominator once (not scaled, no key, no value).  `chunk`: a query sees
         the earlier keys of its own stretch of `chunk` positions, counted from position 0.
+        `keep_first`: the sequence's first so many keys are seen whatever window or chunk says.
         Scores beyond scale times the product: `softcap` c (score <- c tanh(score / c)),
         `slopes` (float32 [num_heads]: slope times the distance to the key comes off),
         `q_temp` (coef, every): the query at position p counts 1 + coef ln(floor((p + 1) /
@@ -735,7 +750,8 @@ class HipOps:
         out = torch.empty_like(q)
         a = AttentionArgs()
         self._fill_attention_args(a, q, out, batch, table, cache, num_heads, num_kv_heads,
-                                  head_dim, scale, window, sink, chunk, softcap, slopes, q_temp)
+                                  head_dim, scale, window, sink, chunk, softcap, slopes, q_temp,
+                                  keep_first)
         extras = softcap is not None or slopes is not None or q_temp is not None
         if (q.dtype == torch.bfloat16 and cache.k_pages.dtype == torch.bfloat16
                 and head_dim % 16 == 0 and head_dim <= 256 and cache.page_size % 4 == 0):
@@ -754,7 +770,7 @@ class HipOps:
     def attend(self, qkv, batch, table, cache, write_cache, *, num_heads, num_kv_heads,
                kv_in_row, head_dim, q_weight, k_weight, eps, cos_sin, scale, window,
                defer_merge=False, sink=None, row_extra=0, chunk=None, softcap=None,
-               slopes=None, q_temp=None):
+               slopes=None, q_temp=None, keep_first=0):
         """Everything between the q/k/v projection and the output projection: per-head
         norm of q and k, rotation, the write of k and v into `cache` (if `write_cache`;
         the row then brings `kv_in_row` = `num_kv_heads` key and value heads) and attention
@@ -776,7 +792,8 @@ class HipOps:
             return self.paged_attention(q, batch, table, cache, num_heads=num_heads,
                                         num_kv_heads=num_kv_heads, head_dim=head_dim,
                                         scale=scale, window=window, sink=sink, chunk=chunk,
-                                        softcap=softcap, slopes=slopes, q_temp=q_temp)
+                                        softcap=softcap, slopes=slopes, q_temp=q_temp,
+                                        keep_first=keep_first)
         # the same argument checks as the preparation kernel's
         qa = self._qk_args(qkv, batch, num_heads=num_heads, kv_in_row=kv_in_row,
                            head_dim=head_dim, q_weight=q_weight, k_weight=k_weight, eps=eps,
@@ -787,9 +804,10 @@ class HipOps:
         out = torch.empty(T, num_heads, head_dim, dtype=qkv.dtype, device=self.device)
         a = AttentionArgs()
         self._fill_attention_args(a, None, out, batch, table, cache, num_heads, num_kv_heads,
-                                  head_dim, scale, window, sink, chunk, softcap, slopes, q_temp)
-        if sink is not None or chunk is not None:
-            defer_merge = False        # the product that merges for itself knows neither
+                                  head_dim, scale, window, sink, chunk, softcap, slopes, q_temp,
+                                  keep_first)
+        if sink is not None or chunk is not None or keep_first:
+            defer_merge = False        # the product that merges for itself knows none of them
         d = AttentionDecodeArgs()
         d.qkv, d.q_weight, d.k_weight = qa.qkv, qa.q_weight, qa.k_weight
         d.cos, d.sin, d.eps, d.kv_in_row = qa.cos, qa.sin, eps, kv_in_row
@@ -846,10 +864,10 @@ class HipOps:
 
     @staticmethod
     def _reach(a):
-        """How many keys a query sees at most (0: all earlier ones), by window and chunk."""
-        if a.window and a.chunk:
-            return min(a.window, a.chunk)
-        return a.window or a.chunk
+        """How many keys a query walks at most (0: all earlier ones), by window and chunk and
+        with the kept first keys in blocks of 64."""
+        reach = min(a.window, a.chunk) if a.window and a.chunk else a.window or a.chunk
+        return reach + -(-a.keep // 64) * 64 if reach else 0
 
     def _attention_mfma(self, a, batch, group, extras=False):
         """Tile the batch's queries (16 rows of q heads x tokens per wavefront), choose how
@@ -964,8 +982,12 @@ class HipOps:
 
     def _fill_attention_args(self, a, q, out, batch, table, cache, num_heads, num_kv_heads,
                              head_dim, scale, window, sink=None, chunk=None, softcap=None,
-                             slopes=None, q_temp=None):
+                             slopes=None, q_temp=None, keep_first=0):
         T = out.shape[0]
+        if keep_first:
+            if int(keep_first) < 0:
+                raise ValueError(f"keep_first={keep_first} must not be negative")
+            a.keep = min(int(keep_first), 1 << 28)     # (further than any sequence goes)
         if chunk is not None:
             if int(chunk) < 1:
                 raise ValueError(f"chunk={chunk} must be positive")
@@ -1067,6 +1089,20 @@ class HipOps:
         """resid += delta / rms(delta) * post_w, in place (float32)."""
         self._postnorm(resid, delta, post_w, eps, None, 0.0, None)
 
+    def postnorm_add_rows(self, resid, delta, post_w, eps, out_dtype):
+        """The same, and the new resid's rows in `out_dtype` (for a sub-layer that reads the
+        stream as it is); float32 rows are the stream itself, not a copy."""
+        if out_dtype == torch.float32:
+            self.postnorm_add(resid, delta, post_w, eps)
+            return resid
+        return self._postnorm(resid, delta, post_w, eps, None, 0.0, out_dtype)
+
+    def stream_rows(self, resid, out_dtype):
+        """The stream's rows in `out_dtype`; float32 rows are the stream itself."""
+        if out_dtype == torch.float32:
+            return resid
+        return self.take_columns(resid, 0, resid.shape[1], out_dtype)
+
     def postnorm_add_norm(self, resid, delta, post_w, post_eps, norm_w, norm_eps, out_dtype):
         """The same, and the norm (norm_w, norm_eps) of the new resid in `out_dtype`."""
         return self._postnorm(resid, delta, post_w, post_eps, norm_w, norm_eps, out_dtype)
@@ -1074,14 +1110,16 @@ class HipOps:
     def _postnorm(self, resid, delta, post_w, post_eps, norm_w, norm_eps, out_dtype):
         delta = self._rows(delta)
         self._check("resid", resid, torch.float32, ndim=2)
-        self._check("delta", delta, torch.float32, shape=resid.shape)
+        self._check("delta", delta, self._FLOATS, shape=resid.shape)
         W = resid.shape[1]
         self._check("post-norm weight", post_w, torch.float32, shape=(W,))
         out = None
         if norm_w is not None:
             self._check("norm weight", norm_w, torch.float32, shape=(W,))
+        if out_dtype is not None:
             out = torch.empty(resid.shape, dtype=out_dtype, device=self.device)
-        self._call(self.lib.ts_postnorm_add, _ptr(resid), _ptr(delta), _ptr(post_w),
+        self._call(self.lib.ts_postnorm_add, _ptr(resid), _ptr(delta), _TYPE_CODE[delta.dtype],
+                   _ptr(post_w),
                    c_float(post_eps), _ptr(norm_w), c_float(norm_eps), _ptr(out),
                    _TYPE_CODE[out_dtype] if out is not None else 0, resid.shape[0], W,
                    self._stream())
@@ -1109,6 +1147,21 @@ class HipOps:
         out = torch.empty(z.shape, dtype=out_dtype, device=self.device)
         self._call(self.lib.ts_polynorm, _ptr(z), _ptr(coef), _ptr(out), _TYPE_CODE[out_dtype],
                    z.shape[0], z.shape[1], c_float(eps), self._stream())
+        return out
+
+    def token_gate(self, z, table, ids, col, out_dtype):
+        """gelu_tanh(z) (z float32 [T, dim]) times columns [col, col + dim) of the tokens' rows
+        of `table` [V, ld]."""
+        self._check("z", z, torch.float32, ndim=2)
+        self._check("token table", table, self._FLOATS, ndim=2)
+        T, dim = z.shape
+        self._check("token ids", ids, torch.int32, shape=(T,))
+        if col < 0 or col + dim > table.shape[1]:
+            raise ValueError(f"token_gate: columns [{col}, {col + dim}) of rows of {table.shape[1]}")
+        out = torch.empty(T, dim, dtype=out_dtype, device=self.device)
+        self._call(self.lib.ts_token_gate, _ptr(z), _ptr(table), _TYPE_CODE[table.dtype], _ptr(ids),
+                   _ptr(out), _TYPE_CODE[out_dtype], T, dim, table.shape[1], int(col),
+                   self._stream())
         return out
 
     # ------------------------------------------------------------ state-space mixer
@@ -1543,35 +1596,61 @@ class HipOps:
         self._call(self.lib.ts_rotate_interleaved, _ptr(x), _TYPE_CODE[x.dtype], _ptr(positions),
                    _ptr(freqs), T, heads, width, offset, dims, self._stream())
 
-    def latent_attention(self, qa, batch, table, cache, *, heads, kv_rank, rot_dim, scale,
-                         window, out_dtype=torch.float32):
-        """Softmax attention of qa [T, heads, kv_rank+rot_dim] (float32) over the latent
-        pages -> sum_t p_t c_t, [T, heads, kv_rank] in `out_dtype`."""
+    def latent_rows(self, rows, batch, table, cache, *, heads, own, kv_rank, rot_dim, kv_norm, eps,
+                    freqs, rot_dims):
+        """Rows [queries: heads x (kv_rank + rot_dim) | kv latent | shared key part] (float32;
+        the last two only with `own`), as one product gives them.  In place: the queries'
+        rotated parts are turned; with `own` the normalised latent and the turned key part are
+        written to the tokens' rows of the latent pages."""
         dl = kv_rank + rot_dim
-        self._check("qa", qa, torch.float32, ndim=3)
+        self._check("rows", rows, torch.float32, ndim=2)
+        T = rows.shape[0]
+        if rows.shape[1] != (heads + int(own)) * dl:
+            raise ValueError(f"latent_rows: rows of {rows.shape[1]} for {heads} heads of {dl}")
+        if own:
+            self._check("kv norm", kv_norm, torch.float32, shape=(kv_rank,))
+        self._check("frequencies", freqs, torch.float32, shape=(rot_dims // 2,))
+        self._check_latent(cache, table, batch, dl)
+        pos, eot, _, _ = self._batch_ptrs(batch, T)
+        self._call(self.lib.ts_latent_rows, _ptr(rows), _ptr(kv_norm if own else None), _ptr(freqs),
+                   _ptr(cache.k_pages), _TYPE_CODE[cache.k_pages.dtype], pos, eot, _ptr(table),
+                   table.shape[1], cache.page_size, T, rows.shape[1], heads, int(own), kv_rank,
+                   rot_dim, rot_dims, c_float(eps), self._stream())
+
+    def latent_attention(self, qa, batch, table, cache, *, heads, kv_rank, rot_dim, scale,
+                         window, out_dtype=torch.float32, sink=None):
+        """Softmax attention of qa [T, heads, kv_rank+rot_dim] (float32; or [T, ld] with the
+        heads' rows side by side and whatever else behind them) over the latent pages ->
+        sum_t p_t c_t, [T, heads, kv_rank] in `out_dtype`.  `sink`: float32 [heads] or None: a
+        score per head that joins the softmax's denominator once (not scaled, no key)."""
+        dl = kv_rank + rot_dim
+        self._check("qa", qa, torch.float32, ndim=qa.dim())
         T = qa.shape[0]
-        if tuple(qa.shape[1:]) != (heads, dl):
+        if tuple(qa.shape[1:]) != (heads, dl) and (qa.dim() != 2 or qa.shape[1] < heads * dl):
             raise ValueError("latent_attention: query shape does not fit")
+        q_ld = qa.numel() // T
+        if sink is not None:
+            self._check("sink", sink, torch.float32, shape=(heads,))
         self._check_latent(cache, table, batch, dl)
         pos, eot, _, _ = self._batch_ptrs(batch, T)
         out = torch.empty(T, heads, kv_rank, dtype=out_dtype, device=self.device)
         if cache.k_pages.dtype == torch.bfloat16 and self.latent_mfma and \
                 self.lib.ts_latent_attention_mfma_fits(kv_rank, rot_dim) == 1:
             self._latent_attention_mfma(qa, out, batch, table, cache, heads, kv_rank, rot_dim,
-                                        scale, window)
+                                        scale, window, q_ld, sink)
             return out
         self._call(self.lib.ts_latent_attention, _ptr(qa), _ptr(cache.k_pages),
                    _TYPE_CODE[cache.k_pages.dtype], _ptr(out), _TYPE_CODE[out_dtype], pos, eot,
                    _ptr(table),
                    table.shape[1], cache.page_size, T, heads, kv_rank, rot_dim,
-                   int(window) if window else 0, c_float(scale), self._stream())
+                   int(window) if window else 0, c_float(scale), q_ld, _ptr(sink), self._stream())
         return out
 
     #: False sends bfloat16 pages to the float32 multiply-add kernel as well
     latent_mfma = True
 
     def _latent_attention_mfma(self, qa, out, batch, table, cache, heads, kv_rank, rot_dim,
-                               scale, window):
+                               scale, window, q_ld, sink):
         """The matrix-core kernel: tiles of 16 (token, head) rows of one entry, made on the
         host once a step and head count; where they are few, each tile's keys are shared out
         over several wavefronts and merged."""
@@ -1616,4 +1695,4 @@ class HipOps:
                    _TYPE_CODE[out.dtype], _ptr(tiles), num_tiles, 4, _ptr(batch.positions),
                    _ptr(table), table.shape[1], cache.page_size, heads, kv_rank, rot_dim,
                    int(window) if window else 0, c_float(scale), per, splits, _ptr(part_o),
-                   _ptr(part_ml), self._stream())
+                   _ptr(part_ml), q_ld, _ptr(sink), self._stream())

@@ -64,6 +64,22 @@ class NormedRows:
     entered: bool
 
 
+@dataclass(frozen=True)
+class RowsAhead:
+    """What a block that reads the stream as it is, without a norm in front, tells the block
+    before it: it wants the stream's rows in the activation dtype, which the kernel that adds
+    the last of the stream can write as it goes."""
+
+
+@dataclass(frozen=True)
+class StreamRows:
+    """The stream summed up (nothing is left to add), with `rows`, the stream in the activation
+    dtype.  Stands where the stream's `delta` does, and only the block that gave the RowsAhead
+    takes it."""
+
+    rows: torch.Tensor
+
+
 class UnmergedRows:
     """What `attend(defer_merge=True)` may return in place of a tensor: a decode step's
     attention output whose key splits have not been merged yet.  It is deliberately no

@@ -159,15 +159,23 @@ class SoftmaxAttention(GroupedQueryAttention):
     key off the score); `q_temp` (coef, every): the query at position n is multiplied by
     1 + coef ln(floor((n + 1) / every) + 1).
 
+    `qk_norm` "plain" (the per-head norms have no weights); `keep_first` (beside its window a
+    query sees the sequence's first so many keys; their pages stay); `wide_output` (the
+    output projection's sums leave in float32, for a block that norms them).
+
     params: prefix, heads, kv_heads, dim, vdim, scale, position (a 'rope_partial' encoding
     of this head_dim, or None), window, qk_norm, qk_norm_eps, sink, gate, own_kv,
-    cache_window, values, bias, chunk, softcap, distance_bias, q_temp."""
+    cache_window, values, bias, chunk, softcap, distance_bias, q_temp, keep_first,
+    wide_output."""
 
     def __init__(self, params, ctx):
         p = dict(params)
         self.dim, self.vdim = int(p["dim"]), int(p["vdim"])
         self.normed = bool(p.get("qk_norm", False)) and p.get("qk_norm") != "projection"
         self.projection_normed = p.get("qk_norm") == "projection"
+        self.plain_normed = p.get("qk_norm") == "plain"
+        self.keep_first = int(p.get("keep_first") or 0)
+        self.wide_output = bool(p.get("wide_output", False))
         self.norm_eps = float(p.get("qk_norm_eps", 0.0))
         self.has_sink, self.has_gate = bool(p.get("sink", False)), bool(p.get("gate", False))
         self.zero_sink, self.head_gate = p.get("sink") == "zero", p.get("gate") == "head"
@@ -189,6 +197,8 @@ class SoftmaxAttention(GroupedQueryAttention):
         self.eps = float(p.get("qk_norm_eps", 0.0)) * self.dim / self.hd
         self.cache_window = p.get("cache_window", self.window)
         self.q_bias = self.o_bias = self.q_proj_norm = self.k_proj_norm = None
+        if self.keep_first and self.window is not None:
+            self.score_options["keep_first"] = self.keep_first
         if p.get("chunk") is not None:
             self.score_options["chunk"] = int(p["chunk"])
         if p.get("softcap") is not None:
@@ -222,7 +232,7 @@ class SoftmaxAttention(GroupedQueryAttention):
             t[pre + "k"] = TensorDecl((self.nkv * self.dim, W))
             if not self.keys_as_values:
                 t[pre + "v"] = TensorDecl((self.nkv * self.vdim, W))
-        if self.normed or self.projection_normed:
+        if (self.normed and not self.plain_normed) or self.projection_normed:
             per = self.nq if self.projection_normed else 1
             t[pre + "q.norm"] = TensorDecl((per * self.dim,), role="vector")
             if self.own_kv:
@@ -240,7 +250,8 @@ class SoftmaxAttention(GroupedQueryAttention):
         return t
 
     def cache_need(self):
-        return PagedKVNeed(self.nkv, self.hd, self.cache_window)
+        return PagedKVNeed(self.nkv, self.hd, self.cache_window,
+                           self.keep_first if self.cache_window is not None else 0)
 
     def load(self, get):
         pre, hd, W = self.prefix, self.hd, self.ctx.width
@@ -301,8 +312,12 @@ class SoftmaxAttention(GroupedQueryAttention):
                 out = torch.zeros(hd, dtype=torch.float32, device=w.device)
                 out[place] = w.float()[src] * (self.dim / hd) ** 0.5
                 return out
-            self.w_qnorm = laid_out(get(pre + "q.norm"))
-            self.w_knorm = laid_out(get(pre + "k.norm")) if self.own_kv else None
+            if self.plain_normed:
+                self.w_qnorm = laid_out(torch.ones(self.dim, device=q.device))
+                self.w_knorm = self.w_qnorm if self.own_kv else None
+            else:
+                self.w_qnorm = laid_out(get(pre + "q.norm"))
+                self.w_knorm = laid_out(get(pre + "k.norm")) if self.own_kv else None
         if self.has_sink:
             self.sink = torch.zeros(self.nq, dtype=torch.float32, device=q.device) \
                 if self.zero_sink else get(pre + "sink").float().contiguous()
@@ -332,12 +347,12 @@ class SoftmaxAttention(GroupedQueryAttention):
                                  self.w_o, resid, hint), resid
 
     def forward(self, h, batch, cache, write_cache):
-        if not (self.has_gate or self.finished or self.o_bias is not None):
+        if not (self.has_gate or self.finished or self.o_bias is not None or self.wide_output):
             return super().forward(h, batch, cache, write_cache)
         rows = self.ops.linear(h, self.w_qkv, torch.float32 if self.finished else self.ctx.dtype)
         out = self.ops.linear(self._gated(self._finish(rows), batch, cache, write_cache),
                               self.w_o, torch.float32 if self.o_bias is not None
-                              else self.ctx.dtype)
+                              or self.wide_output else self.ctx.dtype)
         if self.o_bias is not None:
             self.ops.add_bias(out, self.o_bias)
         return out

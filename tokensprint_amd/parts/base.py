@@ -8,7 +8,7 @@ No part knows which model it is in.
 
 Registries map a `kind` string to a class, one registry per role:
 `MIXERS`, `FEED_FORWARDS`, `NORMS`, `POSITIONS`, `BLOCKS`, `EMBEDDINGS`, `HEADS`,
-`FILTERS`.  A test
+`FILTERS`, `SIDES`.  A test
 or a new architecture adds a part with `register(MIXERS, "my_kind")(MyClass)`.
 """
 
@@ -43,11 +43,13 @@ class TensorDecl:
 
 @dataclass(frozen=True)
 class PagedKVNeed:
-    """Keys and values per token, in pages.  window None = every earlier key."""
+    """Keys and values per token, in pages.  window None = every earlier key; with a window,
+    `keep_first`: the sequence's first so many keys stay as well."""
 
     num_kv_heads: int
     head_dim: int
     window: int | None = None
+    keep_first: int = 0
 
 
 @dataclass(frozen=True)
@@ -206,6 +208,15 @@ class StreamFilter(Part):
         raise NotImplementedError
 
 
+class TokenSide(Part):
+    """What the step's tokens themselves bring into a layer, beside what the stream carries:
+    (the stream's rows in the activation dtype, the step's batch) -> float32 [T, width], which
+    a block norms and adds to the stream."""
+
+    def forward(self, h: torch.Tensor, batch) -> torch.Tensor:
+        raise NotImplementedError
+
+
 class TokenEmbedding(Part):
     """The model's first part: token ids (int32 [T]) -> the residual stream, float32
     [T, width]."""
@@ -292,6 +303,7 @@ BLOCKS: dict[str, type] = {}
 EMBEDDINGS: dict[str, type] = {}
 HEADS: dict[str, type] = {}
 FILTERS: dict[str, type] = {}
+SIDES: dict[str, type] = {}
 
 
 def register(registry: dict[str, type], kind: str, *, replace: bool = False):

@@ -8,8 +8,9 @@ from __future__ import annotations
 
 import torch
 
-from tokensprint_amd.kernels.stream import NormAhead, NormedRows, fused_rmsnorm_of
-from tokensprint_amd.parts.base import (BLOCKS, FEED_FORWARDS, FILTERS, MIXERS, NORMS, Block,
+from tokensprint_amd.kernels.stream import (NormAhead, NormedRows, RowsAhead, StreamRows,
+                                            fused_rmsnorm_of)
+from tokensprint_amd.parts.base import (BLOCKS, FEED_FORWARDS, FILTERS, MIXERS, NORMS, SIDES, Block,
                                         StreamFilter, TensorDecl, SlotStateNeed, register)
 
 
@@ -100,6 +101,60 @@ class SandwichNormBlock(Block):
         out = self.feed_forward.forward(h, batch)
         self._post_add(resid, out, self.ffn_post_norm)
         return resid, None
+
+
+@register(BLOCKS, "post_norm")
+class PostNormBlock(Block):
+    """A norm behind every sub-layer and none in front: the sub-layers read the stream itself,
+    x = x + post(mixer(x)); x = x + post(ffn(x)); then, where the layer has a side input,
+    x = x + post(side(x, tokens)).  Feed-forward and side input may be left out, each with its
+    norm.  The add of a normalised output also writes the rows the next sub-layer (or the next
+    block of this kind) reads; the stream leaves the block summed up (no delta is handed
+    on)."""
+
+    ROLES = {"mixer": (MIXERS, True), "mixer_post_norm": (NORMS, True),
+             "feed_forward": (FEED_FORWARDS, False), "ffn_post_norm": (NORMS, False),
+             "side": (SIDES, False), "side_post_norm": (NORMS, False)}
+
+    def __init__(self, parts, ctx):
+        super().__init__(parts, ctx)
+        if (self.feed_forward is None) != (self.ffn_post_norm is None) or \
+                (self.side is None) != (self.side_post_norm is None):
+            raise ValueError("post_norm: a sub-layer and its norm come together")
+
+    def entry_hint(self):
+        return RowsAhead()
+
+    def _post_add(self, resid, out, post, want_rows):
+        """resid += post(out); the rows of the sum in the activation dtype if wanted."""
+        ops, dtype = self.ctx.ops, self.ctx.dtype
+        fused = fused_rmsnorm_of(post)
+        if fused is None:            # another kind of norm: its own forward, then a plain add
+            ops.stream_add(resid, post.forward(out), None, None)
+            return ops.stream_rows(resid, dtype) if want_rows else None
+        if not want_rows:
+            ops.postnorm_add(resid, out, fused[0], fused[1])
+            return None
+        return ops.postnorm_add_rows(resid, out, fused[0], fused[1], dtype)
+
+    def forward(self, resid, delta, batch, cache, write_cache, next_hint=None):
+        if isinstance(delta, StreamRows):
+            h = delta.rows
+        else:
+            if delta is not None:
+                self.ctx.ops.stream_add(resid, delta, None, None)
+            h = self.ctx.ops.stream_rows(resid, self.ctx.dtype)
+        onward = isinstance(next_hint, RowsAhead)
+        out = self.mixer.forward(h, batch, cache, write_cache)
+        h = self._post_add(resid, out, self.mixer_post_norm,
+                           self.feed_forward is not None or self.side is not None or onward)
+        if self.feed_forward is not None:
+            out = self.feed_forward.forward(h, batch)
+            h = self._post_add(resid, out, self.ffn_post_norm, self.side is not None or onward)
+        if self.side is not None:
+            out = self.side.forward(h, batch)
+            h = self._post_add(resid, out, self.side_post_norm, onward)
+        return resid, StreamRows(h) if onward else None
 
 
 @register(BLOCKS, "parallel_residual")

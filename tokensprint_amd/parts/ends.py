@@ -11,8 +11,8 @@ from __future__ import annotations
 import torch
 
 from tokensprint_amd.kernels.stream import fused_rmsnorm_of
-from tokensprint_amd.parts.base import (EMBEDDINGS, HEADS, OutputHead, SlotStateNeed, TensorDecl,
-                                        TokenEmbedding, register)
+from tokensprint_amd.parts.base import (EMBEDDINGS, HEADS, SIDES, OutputHead, SlotStateNeed,
+                                        TensorDecl, TokenEmbedding, TokenSide, register)
 
 
 @register(EMBEDDINGS, "embedding")
@@ -88,6 +88,45 @@ class BigramEmbedding(TokenEmbedding):
 
     def step_read_tensors(self):
         return [self.norm_w]
+
+
+@register(SIDES, "gated_token_table")
+class GatedTokenTable(TokenSide):
+    """P (gelu_tanh(G h) * e): e is this layer's part of the token's row of a table that holds
+    `dim` columns for each of `parts` layers side by side (columns [index dim, (index + 1) dim)),
+    G [dim, width] reads the stream and P [width, dim] leads back to it.  Tensors: the table,
+    '<prefix>gate', '<prefix>proj'.
+
+    params: prefix, table (tensor name), vocab_size, dim, parts, index."""
+
+    def __init__(self, params, ctx):
+        super().__init__(params, ctx)
+        p = params
+        self.prefix, self.table_name = p["prefix"], p["table"]
+        self.vocab, self.dim = int(p["vocab_size"]), int(p["dim"])
+        self.count, self.index = int(p["parts"]), int(p["index"])
+        if not 0 <= self.index < self.count:
+            raise ValueError(f"{self.prefix}: part {self.index} of {self.count}")
+        self.table = self.w_gate = self.w_proj = None
+
+    def tensors(self):
+        W = self.ctx.width
+        return {self.table_name: TensorDecl((self.vocab, self.count * self.dim)),
+                self.prefix + "gate": TensorDecl((self.dim, W)),
+                self.prefix + "proj": TensorDecl((W, self.dim))}
+
+    def load(self, get):
+        self.table = get(self.table_name)
+        self.w_gate, self.w_proj = get(self.prefix + "gate"), get(self.prefix + "proj")
+
+    def step_read_tensors(self):
+        return [self.w_gate, self.w_proj]       # of the table, the rows of the step's tokens
+
+    def forward(self, h, batch):
+        z = self.ops.linear(h, self.w_gate, torch.float32)
+        act = self.ops.token_gate(z, self.table, batch.token_ids, self.index * self.dim,
+                                  self.ctx.dtype)
+        return self.ops.linear(act, self.w_proj, torch.float32)
 
 
 @register(HEADS, "head")

@@ -15,8 +15,12 @@ from tokensprint_amd.parts.base import FEED_FORWARDS, FeedForward, TensorDecl, r
 
 @register(FEED_FORWARDS, "swiglu")
 class SwiGLU(StreamProducts, FeedForward):
-    """params: prefix, inner_dim, names (the tensors' names behind the prefix, gate, up and
-    down; default 'gate_proj.weight', 'up_proj.weight', 'down_proj.weight')."""
+    """down(silu(gate(h)) * up(h)); with a `limit`, down(g sigmoid(1.702 g) (u + 1)) of g =
+    min(gate(h), limit) and u = up(h) held between -limit and limit.
+
+    params: prefix, inner_dim, names (the tensors' names behind the prefix, gate, up and
+    down; default 'gate_proj.weight', 'up_proj.weight', 'down_proj.weight'), limit (None: the
+    plain unit), wide_output (the result leaves in float32, for a block that norms it)."""
 
     def __init__(self, params, ctx):
         super().__init__(params, ctx)
@@ -24,6 +28,8 @@ class SwiGLU(StreamProducts, FeedForward):
         self.inner = int(params["inner_dim"])
         self.names = tuple(self.prefix + n for n in params.get(
             "names", ("gate_proj.weight", "up_proj.weight", "down_proj.weight")))
+        self.limit = float(params["limit"]) if params.get("limit") is not None else None
+        self.out_dtype = torch.float32 if params.get("wide_output") else ctx.dtype
         self.w_gate_up = self.w_down = None
 
     def tensors(self):
@@ -39,19 +45,22 @@ class SwiGLU(StreamProducts, FeedForward):
         self.w_down = get(self.names[2])
 
     def stream_hint(self, norm):
+        if self.limit is not None:
+            return None          # the products with the norm inside know the plain unit only
         return self.first_product_hint(norm, self.w_gate_up, silu_mul=True)
 
     def forward_from_stream(self, resid, delta, norm, batch, hint=None):
         fused = fused_rmsnorm_of(norm)
-        if fused is None:
+        if fused is None or self.limit is not None:
             return super().forward_from_stream(resid, delta, norm, batch)
         act, resid = self.ops.norm_linear(resid, delta, fused[0], fused[1], self.w_gate_up,
                                           self.ctx.dtype, silu_mul=True)
         return self.last_product(act, self.w_down, resid, hint), resid
 
     def forward(self, h, batch):
-        act = self.ops.linear_silu_mul(h, self.w_gate_up, self.ctx.dtype)
-        return self.ops.linear(act, self.w_down, self.ctx.dtype)
+        form = {} if self.limit is None else {"limit": self.limit}
+        act = self.ops.linear_silu_mul(h, self.w_gate_up, self.ctx.dtype, **form)
+        return self.ops.linear(act, self.w_down, self.out_dtype)
 
 
 @register(FEED_FORWARDS, "polynorm_mlp")

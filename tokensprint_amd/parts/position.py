@@ -47,16 +47,22 @@ class RotaryEncoding(PositionEncoding):
 @register(POSITIONS, "rope_interleaved")
 class InterleavedRotation(PositionEncoding):
     """Rotation of the pairs (2i, 2i+1) of a vector's first `dims` dimensions by the angle
-    position * base^(-2i/dims); the rest passes unchanged.  The pair (u, v) becomes
+    position * base^(-2i/dims); the rest passes unchanged.  With `pairs` "halves" dimension i
+    is paired with i + dims/2 instead: the kernels know neighbours only, so a mixer lays its
+    rotated vectors out by `layout` (a permutation, the same for queries and keys, which
+    changes no score).  The pair (u, v) becomes
     (u cos a - v sin a, v cos a + u sin a).  There is no table and so no longest position:
     kernels take `frequencies()` (float32 [dims/2], rounded once from float64) and compute
     the angle and its cosine and sine in float32 at the position they need.
 
-    params: dims, base."""
+    params: dims, base, pairs ("neighbours", the default, or "halves")."""
 
     def __init__(self, params, ctx):
         super().__init__(params, ctx)
         self.dims = int(params["dims"])
+        self.pairs = params.get("pairs", "neighbours")
+        if self.pairs not in ("neighbours", "halves"):
+            raise ValueError(f"a rotation's pairs are neighbours or halves, not {self.pairs!r}")
         self.base = float(params["base"])
         if self.dims % 2 or self.dims < 2:
             raise ValueError(f"rotated dimensions must be even and at least 2, got {self.dims}")
@@ -66,10 +72,23 @@ class InterleavedRotation(PositionEncoding):
     def frequencies(self):
         return self.freqs
 
+    def layout(self, size: int) -> list[int]:
+        """For a vector of `size` dimensions (the rotated ones first): the given dimension that
+        stands at each place so that a pair's two stand side by side."""
+        if size < self.dims:
+            raise ValueError(f"a rotation of {self.dims} dimensions does not fit {size}")
+        turned = list(range(self.dims))
+        if self.pairs == "halves":
+            half = self.dims // 2
+            turned = [d for i in range(half) for d in (i, i + half)]
+        return turned + list(range(self.dims, size))
+
     def step_read_tensors(self):
         return []
 
     def apply(self, q, k, positions):
+        if self.pairs != "neighbours":
+            raise RuntimeError("vectors whose pairs are halves have to be laid out by `layout`")
         self.ops.rotate_interleaved_inplace(q, positions, self.freqs, self.dims, offset=0)
         if k is not None:
             self.ops.rotate_interleaved_inplace(k, positions, self.freqs, self.dims, offset=0)
