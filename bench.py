@@ -445,6 +445,57 @@ def pinedra_configs(s):
     return config(ff), zolo
 
 
+def fubepel_configs(s):
+    """(Fubepel, Zonopel) at the width, depth, vocabulary and number of matrix parameters of
+    the size `s`.  Fubepel: latent attention (every earlier token visible), gated delta rule,
+    windowed attention that keeps four first tokens, and latent attention that reads the
+    latents of the first layer of the four, in turn; a side input of a head's size in every
+    layer; the feed-forwards' inner size takes up what is left."""
+    import math
+    from tokensprint_amd.weights.random_init import declared_tensors
+    hd, heads, kv = s["head_dim"], s["heads"], s["kv_heads"]
+
+    def layers(ff):
+        latent = {"heads": heads, "dim": hd, "rot_dim": s["rot_dim"], "vdim": hd,
+                  "kv_rank": s["kv_rank"], "scale": (hd + s["rot_dim"]) ** -0.5,
+                  "rot": {"base": 10000.0, "dims": s["rot_dim"]}}
+        sizes = {"heads": heads, "kv_heads": kv, "dim": hd, "vdim": hd}
+        kinds = [("latent_attention", latent), ("delta", dict(sizes, conv=4)),
+                 ("attention", dict(sizes, scale=hd ** -0.5,
+                                    mask={"size": s["window"], "keep_first": 4})),
+                 ("latent_attention", latent)]
+        out = []
+        for i in range(s["layers"]):
+            kind, mixer = kinds[i % 4]
+            mixer = dict(mixer, kv_from=i - 3) if i % 4 == 3 else mixer
+            out.append({"type": kind, "mixer": mixer,
+                        "mlp": {"kind": "dense", "ff": ff, "limit": 7.0}})
+        return out
+
+    def config(ff):
+        return {"architecture": "Fubepel", "width": s["width"], "vocab": s["vocab"],
+                "norm": {"eps": 1e-5}, "embedding": {"scale": 1.0}, "token_side": {"dim": hd},
+                "layers": layers(ff)}
+
+    def count(raw):
+        return sum(math.prod(d.shape) for d in declared_tensors(raw).values())
+    zono = compare_configs(s)[0]
+    spare = count(zono) - count(config(64))
+    ff = 64 + max(0, round(spare / (3 * s["width"] * s["layers"]) / 64)) * 64
+    return config(ff), zono
+
+
+#: design -> (its configuration and that of the closest design at equal size, that design)
+COMPARISONS = {"zonopel": (compare_configs, "qwen3"), "palelix": (palelix_configs, "zonopel"),
+               "zolorax": (zolorax_configs, "zonopel"), "pinedra": (pinedra_configs, "zolorax"),
+               "fubepel": (fubepel_configs, "zonopel")}
+
+
+def chosen_design(args, what):
+    """The design whose --compare-... or --profile-... option is given, or None."""
+    return next((d for d in COMPARISONS if getattr(args, f"{what}_{d}")), None)
+
+
 class TimedOps:
     """Wraps a kernel provider: every call of one of its operations is bracketed by events,
     and `seconds` sums them per operation name (an eager step's kernels, one by one)."""
@@ -504,21 +555,17 @@ def op_times(model, page, entries_of, reps=3):
     return runs[len(runs) // 2]
 
 
-def zonopel_profile_step(args) -> int:
-    """Four eager steps of the Zonopel (or, `--profile-palelix`, the Palelix) model of
-    `--compare-size` (default 1b-layers): a 2,048-token prompt, or a decode step of eight
+def profile_step(args) -> int:
+    """Four eager steps of the model whose --profile-... option is given, at `--compare-size` (default 1b-layers): a 2,048-token prompt, or a decode step of eight
     requests at 2,048 tokens; for a profiler."""
     import torch
     from tokensprint_amd.engine.assemble import random_model
     from tokensprint_amd.engine.runner import ModelRunner
     size = COMPARE_SIZES[args.compare_size or "1b-layers"]
-    zono = palelix_configs(size)[0] if args.profile_palelix else \
-        zolorax_configs(size)[0] if args.profile_zolorax else \
-        pinedra_configs(size)[0] if args.profile_pinedra else compare_configs(size)[0]
-    args.profile_zonopel = args.profile_zonopel or args.profile_palelix or args.profile_zolorax \
-        or args.profile_pinedra
-    _, model = random_model(zono, 0, args.dtype, "cuda:0")
-    make = prefill_entries(2048) if args.profile_zonopel == "prefill" else decode_entries(8, 2048)
+    design = chosen_design(args, "profile")
+    profiled = getattr(args, f"profile_{design}")
+    _, model = random_model(COMPARISONS[design][0](size)[0], 0, args.dtype, "cuda:0")
+    make = prefill_entries(2048) if profiled == "prefill" else decode_entries(8, 2048)
     lengths = make(None)
     runner = ModelRunner(model, page_size=16, num_pages=sum(-(-n // 16) + 1 for n in lengths),
                          num_slots=len(lengths))
@@ -527,30 +574,27 @@ def zonopel_profile_step(args) -> int:
         batch.plans.clear()
         runner.run(batch)
     torch.cuda.synchronize()
-    print(json.dumps({"profiled": args.profile_zonopel, "steps": 4}))
+    print(json.dumps({"profiled": profiled, "steps": 4}))
     return 0
 
 
-def zonopel_compare(args) -> int:
-    """Prefill and decode throughput of Zonopel beside Qwen3 at equal sizes, and the time of
-    every kind of kernel in a 2,048-token prompt and in a decode step of eight requests.
+def compare_designs(args) -> int:
+    """Prefill and decode throughput of the design whose --compare-... option is given beside
+    the closest other design at equal sizes, and the time of every kind of kernel in a 2,048-token prompt and in a decode step of eight requests.
     Prints one JSON line of its own."""
     import torch
     from tokensprint_amd.engine.assemble import random_model
     page, T, b, ctx = 16, 2048, 8, 2048
-    pair = ("palelix", "zonopel") if args.compare_palelix else \
-        ("zolorax", "zonopel") if args.compare_zolorax else \
-        ("pinedra", "zolorax") if args.compare_pinedra else ("zonopel", "qwen3")
+    design = chosen_design(args, "compare")
+    pair = (design, COMPARISONS[design][1])
     out = {"metric": f"{pair[0]} beside {pair[1]} at equal sizes (random weights, bf16)",
            "sizes": {}}
     for name, size in COMPARE_SIZES.items():
         if args.compare_size and name != args.compare_size:
             continue
         row = {}
-        configs = palelix_configs(size) if args.compare_palelix else \
-            zolorax_configs(size) if args.compare_zolorax else \
-            pinedra_configs(size) if args.compare_pinedra else compare_configs(size)
-        for design, raw in zip(pair, configs):
+        configs = COMPARISONS[design][0](size)
+        for kind, raw in zip(pair, configs):
             _, model = random_model(raw, 0, args.dtype, "cuda:0")
             vocab = size["vocab"]
             _, engine = make_engine(raw, args.dtype, None, 1, 4096, T, page, model=model)
@@ -563,7 +607,7 @@ def zonopel_compare(args) -> int:
             del engine
             params = sum(t.numel() for part in model.parts() for t in part.held_tensors()
                          if t.dim() == 2)
-            row[design] = {
+            row[kind] = {
                 "matrix_params_m": round(params / 1e6, 1),
                 "prefill_tok_s": round(T / pre, 1), "prefill_ms": round(pre * 1e3, 3),
                 "decode_tok_s": round(decoded / sec, 1),
@@ -611,6 +655,11 @@ def main() -> int:
     ap.add_argument("--compare-pinedra", action="store_true",
                     help="instead of the benchmark: prefill and decode throughput of Pinedra "
                          "beside Zolorax at equal sizes, with the time of every kind of kernel")
+    ap.add_argument("--compare-fubepel", action="store_true",
+                    help="instead of the benchmark: prefill and decode throughput of Fubepel "
+                         "beside Zonopel at equal sizes, with the time of every kind of kernel")
+    ap.add_argument("--profile-fubepel", default=None, choices=["prefill", "decode"],
+                    help="as --profile-zonopel, for the Fubepel model of --compare-size")
     ap.add_argument("--profile-pinedra", default=None, choices=["prefill", "decode"],
                     help="as --profile-zonopel, for the Pinedra model of --compare-size")
     ap.add_argument("--profile-zolorax", default=None, choices=["prefill", "decode"],
@@ -629,10 +678,10 @@ def main() -> int:
     import torch
     from tokensprint_amd.config import load_named_config
 
-    if args.profile_zonopel or args.profile_palelix or args.profile_zolorax or args.profile_pinedra:
-        return zonopel_profile_step(args)
-    if args.compare_zonopel or args.compare_palelix or args.compare_zolorax or args.compare_pinedra:
-        return zonopel_compare(args)
+    if chosen_design(args, "profile"):
+        return profile_step(args)
+    if chosen_design(args, "compare"):
+        return compare_designs(args)
     raw = load_named_config(args.model)
     full_layers = raw["num_hidden_layers"]
     layers = args.layers or full_layers

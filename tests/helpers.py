@@ -468,3 +468,98 @@ def write_pinedra_model(folder, cfg, seed, dtype, std=0.2, sharpen=3.0, router=4
             tensors[name] = (tensors[name].float() * factor).to(tensors[name].dtype)
     save_file(tensors, str(file))
     return d
+
+
+# ------------------------------------------------------------------ Fubepel
+
+
+def fubepel_dense(ff, limit):
+    return {"kind": "dense", "ff": ff, "limit": limit}
+
+
+def fubepel_delta(*, heads, kv_heads, dim, vdim, conv, mlp=None):
+    return {"type": "delta", "mlp": mlp, "mixer": {"heads": heads, "kv_heads": kv_heads,
+                                                   "dim": dim, "vdim": vdim, "conv": conv}}
+
+
+def fubepel_attention(*, heads, kv_heads, dim, vdim, scale, window, keep_first, mlp=None):
+    mixer = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "scale": scale}
+    if window is not None:
+        mixer["mask"] = {"size": window, "keep_first": keep_first}
+    return {"type": "attention", "mixer": mixer, "mlp": mlp}
+
+
+def fubepel_latent(*, heads, dim, rot_dim, vdim, kv_rank, scale, base, kv_from=None, mlp=None):
+    mixer = {"heads": heads, "dim": dim, "rot_dim": rot_dim, "vdim": vdim, "kv_rank": kv_rank,
+             "scale": scale, "rot": {"base": base, "dims": rot_dim}}
+    if kv_from is not None:
+        mixer["kv_from"] = kv_from
+    return {"type": "latent_attention", "mixer": mixer, "mlp": mlp}
+
+
+def fubepel_config(*, width, vocab, eps, embed_scale, side_dim, layers):
+    cfg = {"architecture": "Fubepel", "width": width, "vocab": vocab, "norm": {"eps": eps},
+           "embedding": {"scale": embed_scale}, "layers": layers}
+    if side_dim is not None:
+        cfg["token_side"] = {"dim": side_dim}
+    return cfg
+
+
+# Three small models that differ in every size and option: each mixer first, in the middle and
+# last; latents of its own, read by one later layer and by two, the reader with other heads,
+# scale and value size; windows below a page, of several pages, of a single token and none;
+# kept first tokens fewer than a page, more than a page, more than the window, one and none;
+# one key/value head, several, and as many as query heads; value sizes above, below and equal
+# to the key size; one to four taps; limits that clamp nearly everything and nearly nothing;
+# layers without a feed-forward; a model without a side input; embedding scales of 1 and
+# others; rotated parts of 2 dimensions and of more than the unrotated ones.
+FUBE_A = fubepel_config(
+    width=40, vocab=97, eps=1e-5, embed_scale=2.5, side_dim=6, layers=[
+        fubepel_latent(heads=3, dim=8, rot_dim=4, vdim=10, kv_rank=20, scale=0.4, base=10000.0,
+                       mlp=fubepel_dense(24, 0.7)),
+        fubepel_attention(heads=4, kv_heads=2, dim=12, vdim=20, scale=0.6, window=3, keep_first=2,
+                          mlp=fubepel_dense(20, 3.0)),
+        fubepel_delta(heads=4, kv_heads=2, dim=8, vdim=12, conv=3, mlp=None),
+        fubepel_latent(heads=2, dim=16, rot_dim=4, vdim=6, kv_rank=20, scale=0.25, base=10000.0,
+                       kv_from=0, mlp=fubepel_dense(12, 7.0)),
+    ])
+FUBE_B = fubepel_config(
+    width=72, vocab=131, eps=3e-6, embed_scale=1.0, side_dim=16, layers=[
+        fubepel_attention(heads=6, kv_heads=1, dim=24, vdim=16, scale=0.25, window=37, keep_first=21,
+                          mlp=fubepel_dense(40, 1.5)),
+        fubepel_latent(heads=5, dim=4, rot_dim=16, vdim=12, kv_rank=32, scale=0.08, base=500.0, mlp=None),
+        fubepel_delta(heads=3, kv_heads=3, dim=16, vdim=8, conv=1, mlp=fubepel_dense(32, 0.3)),
+        fubepel_latent(heads=5, dim=12, rot_dim=16, vdim=8, kv_rank=32, scale=0.06, base=500.0,
+                       kv_from=1, mlp=fubepel_dense(48, 2.0)),
+        fubepel_latent(heads=1, dim=8, rot_dim=16, vdim=24, kv_rank=32, scale=0.1, base=500.0,
+                       kv_from=1, mlp=fubepel_dense(16, 1.0)),
+        fubepel_latent(heads=2, dim=16, rot_dim=2, vdim=16, kv_rank=30, scale=0.07, base=100.0,
+                       mlp=fubepel_dense(24, 5.0)),
+    ])
+FUBE_C = fubepel_config(
+    width=32, vocab=64, eps=1e-4, embed_scale=6.0, side_dim=None, layers=[
+        fubepel_delta(heads=6, kv_heads=2, dim=4, vdim=16, conv=4, mlp=fubepel_dense(16, 1.2)),
+        fubepel_attention(heads=3, kv_heads=3, dim=16, vdim=16, scale=0.4, window=1, keep_first=9,
+                          mlp=fubepel_dense(24, 0.5)),
+        fubepel_attention(heads=2, kv_heads=2, dim=8, vdim=32, scale=0.7, window=None, keep_first=0,
+                          mlp=None),
+        fubepel_attention(heads=4, kv_heads=1, dim=32, vdim=8, scale=0.3, window=50, keep_first=1,
+                          mlp=fubepel_dense(8, 4.0)),
+    ])
+FUBE = {"A": (FUBE_A, 75, 4), "B": (FUBE_B, 74, 16), "C": (FUBE_C, 73, 8)}   # cfg, seed, page
+
+
+def write_fubepel_model(folder, cfg, seed, dtype, std=0.2, sharpen=3.0):
+    """Random weights, then the latent attention's query weights scaled up (`sharpen`), so that
+    its softmax weighs few keys heavily and a key that is lost or seen too early shows (the
+    windowed attention's queries and keys are normed: its scores are given by its scale)."""
+    from safetensors.torch import load_file, save_file
+    from tokensprint_amd.weights import write_random_model
+    d = write_random_model(folder, cfg, seed, dtype, std=std)
+    file = next(d.glob("*.safetensors"))
+    tensors = load_file(str(file))
+    for name in tensors:
+        if name.endswith(".mix.uk"):
+            tensors[name] = (tensors[name].float() * sharpen).to(tensors[name].dtype)
+    save_file(tensors, str(file))
+    return d

@@ -112,3 +112,22 @@ def test_zolorax_and_zonopel_are_compared_at_equal_size():
         assert {e["type"] for e in zolo["layers"]} == {"rglru", "attention"}
         assert any("kv_from" in e["mixer"] for e in zolo["layers"])
         assert {e["mlp"]["kind"] for e in zolo["layers"]} == {"dense", "moe"}
+
+
+def test_fubepel_and_zonopel_are_compared_at_equal_size():
+    """`bench.py --compare-fubepel` builds a Fubepel and a Zonopel configuration per size with
+    the same width, depth, vocabulary and (within 2 %) number of parameters, every kind of
+    mixer and a layer that reads another's latents."""
+    import math
+
+    import bench
+    from tokensprint_amd.weights.random_init import declared_tensors
+    for name, size in bench.COMPARE_SIZES.items():
+        fube, zono = bench.fubepel_configs(size)
+        count = [sum(math.prod(d.shape) for d in declared_tensors(raw).values())
+                 for raw in (fube, zono)]
+        assert abs(count[0] - count[1]) <= 0.02 * count[0], (name, count)
+        assert fube["width"] == zono["width"] and fube["vocab"] == zono["vocab"]
+        assert len(fube["layers"]) == len(zono["layers"])
+        assert {e["type"] for e in fube["layers"]} == {"latent_attention", "delta", "attention"}
+        assert any("kv_from" in e["mixer"] for e in fube["layers"]) and fube["token_side"]

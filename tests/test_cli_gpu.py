@@ -202,3 +202,23 @@ def test_run_py_serves_a_pinedra_model(gpu_device, tmp_path):
     for _ in range(9):
         tokens.append(int(pinedra_plain.forward(pcfg, w, tokens)[-1].argmax()))
     assert got == tokens[len(prompt):]
+
+
+def test_run_py_serves_a_fubepel_model(gpu_device, tmp_path):
+    """The same for Fubepel: kept first tokens, a layer that reads another's latents, a
+    recurrence and a side input of every token."""
+    from helpers import FUBE_A
+    from plain import fubepel_plain
+    prompt = random_prompt(21, FUBE_A["vocab"], 9)
+    model_dir = tmp_path / "fube-a"
+    proc = run_program(["run.py", "--config-json", config_json(tmp_path, FUBE_A),
+                        "--random-weights", "2", "--model-dir", model_dir, "--dtype", "float32",
+                        "--temperature", "0", "--max-tokens", "9", "--ignore-eos", "True",
+                        "--max-num-seqs", "8", "--max-model-len", "256",
+                        "--prompt-ids", ",".join(map(str, prompt))])
+    got = json.loads(proc.stdout.strip().splitlines()[-1])
+    pcfg, w = fubepel_plain.read_model_dir(model_dir)
+    tokens = list(prompt)
+    for _ in range(9):
+        tokens.append(int(fubepel_plain.forward(pcfg, w, tokens)[-1].argmax()))
+    assert got == tokens[len(prompt):]

@@ -336,9 +336,11 @@ extern "C" int ts_latent_attention(const float* qa, const void* pages, int cache
 // S^T[key 4g + t][row r], which is, in place, its part of the second product's B operand;
 // its softmax statistics are shared with lanes r + 16, r + 32, r + 48; its part of O^T is
 // [columns 16 db + 4g + t][row r], so rescaling needs nothing from other lanes.
-// Keys are walked in blocks of 32 at absolute multiples of 32.  Where a step has few
-// tiles, a tile's keys are shared out in runs of `keys_per_split` over several wavefronts,
-// whose unnormalised results and statistics a second kernel merges.
+// Keys are walked in blocks of 32 at absolute multiples of 32, staged in LDS, from where both
+// operands come: the K operand as 16 bytes of a row, the C^T operand by the transposing read.
+// Where a step has few tiles, a tile's keys are shared out in runs of `keys_per_split` over
+// several workgroups, whose unnormalised results and statistics (the largest score in units
+// of log2) a second kernel merges.
 typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8_l;
 
 struct LatentMfmaArgs {
@@ -359,158 +361,336 @@ struct LatentMfmaArgs {
 
 constexpr int kLatentPad = 8;     // elements between staged rows: operand reads spread over banks
 
-// The wavefronts of a workgroup take consecutive tiles of one entry (where keys are shared
-// out, one tile and three empty ones, which only help load) and walk the union of their
-// keys together: each block of
-// 32 cached rows is staged in LDS once by all of them (16-byte loads, rows that are not
-// there as zeros), and both operands come from there: the K operand as 16 bytes of a row,
-// the C^T operand as eight 2-byte reads of a column.  A tile with no rows only helps load.
+// The query operand of a row: elements 32 s + 8 g .. + 7.  (The row's length is a multiple of
+// 8: eight elements are there together or not at all.)
+template <int KS>
+__device__ __forceinline__ void load_query_row(bf16x8_l (&q)[KS], const float* qr, int dl, int g) {
+#pragma unroll
+  for (int s = 0; s < KS; ++s) {
+    const int d0 = 32 * s + 8 * g;
+    const float* src = qr + min(d0, dl - 8);
+    const f32x4_l lo4 = *(const f32x4_l*)src, hi4 = *(const f32x4_l*)(src + 4);
+    const bool there = d0 < dl;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      q[s][j] = (__bf16)(there ? lo4[j] : 0.f);
+      q[s][4 + j] = (__bf16)(there ? hi4[j] : 0.f);
+    }
+  }
+}
+
+// Scores, in units of log2, of row r with keys kb + 16 (e / 4) + 4 g + e % 4, the keys staged
+// as rows of `stride` elements at k_s; -inf where the row does not see a key.  Returns the
+// largest of the row's 32.
+template <int KS>
+__device__ __forceinline__ float score_block(float (&sc)[8], const bf16x8_l (&q)[KS],
+                                             const bf16_t* k_s, int stride, int kb, int dl,
+                                             float scale_log2, int pos, int lo, int r, int g) {
+  // two blocks of 16 keys, the reduction over the row in two chains each
+  f32x4_l st[2][2];
+#pragma unroll
+  for (int c = 0; c < 4; ++c) st[c / 2][c % 2] = f32x4_l{0.f, 0.f, 0.f, 0.f};
+  const bf16_t* kr = k_s + r * stride + 8 * g;
+#pragma unroll
+  for (int s = 0; s < KS; ++s) {
+    if (32 * s < dl) {
+      // (past the row's end the query's elements are zeros: the row's last eight stand in)
+      const int d0 = min(32 * s, dl - 8 - 8 * g);
+#pragma unroll
+      for (int blk = 0; blk < 2; ++blk) {
+        const bf16x8_l kop = *(const bf16x8_l*)(kr + 16 * blk * stride + d0);
+        st[blk][s & 1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kop, q[s], st[blk][s & 1], 0, 0, 0);
+      }
+    }
+  }
+  float mx = -INFINITY;
+#pragma unroll
+  for (int e = 0; e < 8; ++e) {
+    const int key = kb + 16 * (e / 4) + 4 * g + e % 4;
+    const float dot = st[e / 4][0][e % 4] + st[e / 4][1][e % 4];
+    sc[e] = (key <= pos && key >= lo) ? dot * scale_log2 : -INFINITY;
+    mx = fmaxf(mx, sc[e]);
+  }
+  mx = fmaxf(mx, __shfl_xor(mx, 16, kWave));
+  return fmaxf(mx, __shfl_xor(mx, 32, kWave));
+}
+
+// Weights of the block's scores relative to m_use; returns this lane's share of their sum.
+__device__ __forceinline__ float weigh_block(bf16x8_l& pv, const float (&sc)[8], float m_use) {
+  float sum = 0.f;
+#pragma unroll
+  for (int e = 0; e < 8; ++e) {
+    const float p = __builtin_amdgcn_exp2f(sc[e] - m_use);
+    sum += p;
+    pv[e] = (__bf16)p;
+  }
+  return sum;
+}
+
+// O^T += C^T P^T for `DB` blocks of 16 columns from `db0` on.  A lane's column of four keys
+// comes out of LDS by the transposing read (sixteen lanes name four rows' runs of sixteen
+// elements, four elements a lane, and each gets one column of the four rows; columns from
+// kv_rank on, which belong to the key part or the padding, give results that nobody stores).
+template <int DB>
+__device__ __forceinline__ void value_block(f32x4_l (&o)[DB], bf16x8_l pv, const bf16_t* k_s,
+                                            int stride, int kv_rank, int db0, int r, int g) {
+  typedef short s16x4 __attribute__((ext_vector_type(4)));
+  typedef __attribute__((address_space(3))) s16x4* Lds4;
+  const bf16_t* vrow = k_s + (4 * g + r / 4) * stride + 4 * (r % 4) + 16 * db0;
+#pragma unroll
+  for (int db = 0; db < DB; ++db) {
+    if (16 * (db0 + db) < kv_rank) {
+      const s16x4 a = __builtin_amdgcn_ds_read_tr16_b64_v4i16((Lds4)(vrow + 16 * db));
+      const s16x4 b = __builtin_amdgcn_ds_read_tr16_b64_v4i16((Lds4)(vrow + 16 * stride + 16 * db));
+      const auto both = __builtin_shufflevector(a, b, 0, 1, 2, 3, 4, 5, 6, 7);
+      o[db] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_l, both), pv,
+                                                      o[db], 0, 0, 0);
+    }
+  }
+}
+
+// The four lanes r, r + 16, r + 32, r + 48 hold a row: the sum of their shares.
+__device__ __forceinline__ float row_total(float v) {
+  v += __shfl_xor(v, 16, kWave);
+  return v + __shfl_xor(v, 32, kWave);
+}
+
+// A sink's weight relative to `m_log2`, a largest score in units of log2.
+__device__ __forceinline__ float sink_weight_log2(float sink, float m_log2) {
+  return __builtin_amdgcn_exp2f(fminf(sink * 1.44269504088896f - m_log2, 100.f));
+}
+
+// Many tiles: the four wavefronts of a workgroup take four tiles of one entry (the last of an
+// entry's may be empty: such a wavefront only helps load) and walk the union of their keys
+// together.  Each block of 32 cached rows passes through registers into one of two LDS
+// buffers, eight threads a row, sent for while the block before it is worked on; the page of
+// the block after that is looked up meanwhile.
 template <int KS, int DB, typename TO>
 __global__ __launch_bounds__(4 * kWave) void latent_attention_mfma_kernel(LatentMfmaArgs a) {
+  constexpr int PIECES = (4 * KS + 7) / 8;                // 16-byte pieces of a row a thread brings
   extern __shared__ __attribute__((aligned(16))) unsigned char lds_raw[];
   const int dl = a.kv_rank + a.rot_dim, P = a.page_size;
   const int stride = dl + kLatentPad;
-  bf16_t* k_s = (bf16_t*)lds_raw;                         // [32][stride]
-  int* krow_s = (int*)(lds_raw + (size_t)32 * stride * sizeof(bf16_t));   // [32]
-  const int waves = blockDim.x / kWave, wave = threadIdx.x / kWave;
-  const int lane = threadIdx.x % kWave, r = lane % 16, g = lane / 16;
-  const int tile0 = blockIdx.x * waves, tile = tile0 + wave, split = blockIdx.y;
+  bf16_t* bufs = (bf16_t*)lds_raw;                        // [2][32][stride]
+  const int wave = threadIdx.x / kWave, lane = threadIdx.x % kWave, r = lane % 16, g = lane / 16;
+  const int tile0 = blockIdx.x * 4, tile = tile0 + wave;
   const int row0 = a.tiles[3 * tile], nrows = a.tiles[3 * tile + 1];
   const int* tab = a.table + (int64_t)a.tiles[3 * tile0 + 2] * a.table_width;
   const bool row_ok = r < nrows;
   const int my_row = row0 + max(0, min(r, nrows - 1));
-  const int pos_r = a.positions[my_row / a.heads];
+  const int my_head = my_row % a.heads, my_token = my_row / a.heads;
+  const int pos_r = a.positions[my_token];
+  const int my_pos = row_ok ? pos_r : -1;
   const int lo_r = a.window > 0 ? max(0, pos_r - a.window + 1) : 0;
   // the keys of the whole workgroup: from the first tile's first token to the last token
   const int pos_first = a.positions[a.tiles[3 * tile0] / a.heads];
   const int lo_t = a.window > 0 ? max(0, pos_first - a.window + 1) : 0;
   int hi_t = pos_first;
-  for (int w = 0; w < waves; ++w) {
+  for (int w = 0; w < 4; ++w) {
     const int n = a.tiles[3 * (tile0 + w) + 1];
     if (n > 0) hi_t = max(hi_t, a.positions[(a.tiles[3 * (tile0 + w)] + n - 1) / a.heads]);
   }
-  const int k_begin = (lo_t / 32) * 32 + split * a.keys_per_split;
-  const int k_end = min(k_begin + a.keys_per_split, hi_t + 1);
+  const int k_begin = (lo_t / 32) * 32, k_end = hi_t + 1;
+  // the wavefront's own first and last visible keys: blocks outside are not its business
+  const int tile_last = __builtin_amdgcn_readfirstlane(nrows) > 0
+      ? a.positions[(row0 + nrows - 1) / a.heads] : -1;
+  const int tile_lo = __builtin_amdgcn_readfirstlane(a.window > 0
+      ? max(0, a.positions[row0 / a.heads] - a.window + 1) : 0);
 
+  const int key_l = threadIdx.x / 8, piece = threadIdx.x % 8;
+  const int parts = dl / 8;
+  auto look_up = [&](int kb) {
+    const int j = kb + key_l;
+    return (j >= lo_t && j <= hi_t) ? tab[j / P] : -1;
+  };
+  bf16x8_l held[PIECES];
+  auto fetch = [&](int kb, int page) {
+    const bf16_t* row = a.pages + ((int64_t)max(page, 0) * P + (kb + key_l) % P) * dl;
+#pragma unroll
+    for (int i = 0; i < PIECES; ++i) held[i] = *(const bf16x8_l*)(row + 8 * min(piece + 8 * i, parts - 1));
+  };
+  auto commit = [&](bf16_t* buf, int page) {
+    const bf16x8_l zero = {0, 0, 0, 0, 0, 0, 0, 0};
+#pragma unroll
+    for (int i = 0; i < PIECES; ++i)
+      if (piece + 8 * i < parts)
+        *(bf16x8_l*)(buf + key_l * stride + 8 * (piece + 8 * i)) = page >= 0 ? held[i] : zero;
+  };
+  int page = look_up(k_begin), page_next = look_up(k_begin + 32);
+  fetch(k_begin, page);
   bf16x8_l q[KS];
-  const int my_head = my_row % a.heads;
-  const float* qr = a.qa + (int64_t)(my_row / a.heads) * a.q_ld + my_head * dl;
-#pragma unroll
-  for (int s = 0; s < KS; ++s) {
-    const int d0 = 32 * s + 8 * g;
-#pragma unroll
-    for (int j = 0; j < 8; ++j) q[s][j] = (d0 + j < dl) ? (__bf16)qr[d0 + j] : (__bf16)0.f;
-  }
+  load_query_row<KS>(q, a.qa + (int64_t)my_token * a.q_ld + my_head * dl, dl, g);
   f32x4_l o[DB];
 #pragma unroll
   for (int db = 0; db < DB; ++db) o[db] = f32x4_l{0.f, 0.f, 0.f, 0.f};
-  float m = -INFINITY, l = 0.f;
-  const int parts = dl / 8;
-
-  for (int kb = k_begin; kb < k_end; kb += 32) {
-    __syncthreads();                      // the block before has been used by everyone
-    for (int c = threadIdx.x; c < 32 * parts; c += blockDim.x) {
-      const int key = c / parts, part = c % parts;
-      const int j = kb + key;
-      int page = -1;
-      if (j >= lo_t && j <= hi_t) page = tab[j / P];
-      const int row = page >= 0 ? page * P + j % P : -1;
-      bf16x8_l v;
-      if (row >= 0) v = *(const bf16x8_l*)(a.pages + (int64_t)row * dl + part * 8);
-      else {
-#pragma unroll
-        for (int j8 = 0; j8 < 8; ++j8) v[j8] = (__bf16)0.f;
-      }
-      *(bf16x8_l*)(k_s + key * stride + part * 8) = v;
-      if (part == 0) krow_s[key] = row;
+  float m = -INFINITY, l = 0.f;            // l: this lane's share of the row's sum
+  commit(bufs, page);
+  __syncthreads();
+  const float scale_log2 = a.scale * 1.44269504088896341f;
+  int which = 0;
+  for (int kb = k_begin; kb < k_end; kb += 32, which ^= 1) {
+    const bool more = kb + 32 < k_end;
+    if (more) {
+      page = page_next;
+      fetch(kb + 32, page);
+      page_next = look_up(kb + 64);
     }
+    if (kb <= tile_last && kb + 31 >= tile_lo) {
+      const bf16_t* k_s = bufs + which * 32 * stride;
+      float sc[8];
+      bf16x8_l pv;
+      const float m_new = fmaxf(m, score_block<KS>(sc, q, k_s, stride, kb, dl, scale_log2, my_pos, lo_r, r, g));
+      // (a finite stand-in while the row has seen no key makes every exponential zero)
+      const float m_use = fmaxf(m_new, -1e30f);
+      const float corr = __builtin_amdgcn_exp2f(m - m_use);
+      l = l * corr + weigh_block(pv, sc, m_use);
+      m = m_new;
+      if (__builtin_amdgcn_ballot_w64(corr != 1.f) != 0) {
+#pragma unroll
+        for (int db = 0; db < DB; ++db) o[db] = o[db] * corr;
+      }
+      value_block<DB>(o, pv, k_s, stride, a.kv_rank, 0, r, g);
+    }
+    if (more) commit(bufs + (which ^ 1) * 32 * stride, page);
     __syncthreads();
-    if (__builtin_amdgcn_readfirstlane(nrows) <= 0) continue;   // an empty tile only loads
-    f32x4_l st[2];
-#pragma unroll
-    for (int blk = 0; blk < 2; ++blk) {
-      const bf16_t* kr = k_s + (16 * blk + r) * stride;
-      st[blk] = f32x4_l{0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-      for (int s = 0; s < KS; ++s) {
-        const int d0 = 32 * s + 8 * g;
-        if (32 * s < dl) {
-          bf16x8_l kop;
-          if (d0 + 8 <= dl) kop = *(const bf16x8_l*)(kr + d0);
-          else {
-#pragma unroll
-            for (int j8 = 0; j8 < 8; ++j8) kop[j8] = (__bf16)0.f;
-          }
-          st[blk] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kop, q[s], st[blk], 0, 0, 0);
-        }
-      }
-    }
-    float sc[8];
-    float mx = -INFINITY;
-#pragma unroll
-    for (int e = 0; e < 8; ++e) {
-      const int blk = e / 4, t = e % 4;
-      const int key = kb + 16 * blk + 4 * g + t;
-      const bool vis = row_ok && krow_s[16 * blk + 4 * g + t] >= 0 && key <= pos_r && key >= lo_r;
-      sc[e] = vis ? st[blk][t] * a.scale : -INFINITY;
-      mx = fmaxf(mx, sc[e]);
-    }
-    mx = fmaxf(mx, __shfl_xor(mx, 16, kWave));
-    mx = fmaxf(mx, __shfl_xor(mx, 32, kWave));
-    const float m_new = fmaxf(m, mx);
-    const float corr = m_new == -INFINITY ? 1.f : expf(m - m_new);
-    bf16x8_l pv;
-    float psum = 0.f;
-#pragma unroll
-    for (int e = 0; e < 8; ++e) {
-      const float p = sc[e] == -INFINITY ? 0.f : expf(sc[e] - m_new);
-      psum += p;
-      pv[e] = (__bf16)p;
-    }
-    psum += __shfl_xor(psum, 16, kWave);
-    psum += __shfl_xor(psum, 32, kWave);
-    l = l * corr + psum;
-    m = m_new;
-    const bf16_t* vcol = k_s + (4 * g) * stride + r;
-#pragma unroll
-    for (int db = 0; db < DB; ++db) {
-      if (16 * db < a.kv_rank) {
-        bf16x8_l vop;
-#pragma unroll
-        for (int e = 0; e < 8; ++e)
-          vop[e] = vcol[(16 * (e / 4) + e % 4) * stride + 16 * db];
-        o[db] = o[db] * corr;
-        o[db] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vop, pv, o[db], 0, 0, 0);
-      }
-    }
   }
-  if (a.splits == 1) {
-    if (!row_ok) return;
-    if (a.sink) l += sink_weight(a.sink[my_head], m);
-    const float inv = l > 0.f ? 1.0f / l : 0.f;
-    TO* orow = (TO*)a.out + (int64_t)my_row * a.kv_rank;
-#pragma unroll
-    for (int db = 0; db < DB; ++db)
-#pragma unroll
-      for (int t = 0; t < 4; ++t) {
-        const int d = 16 * db + 4 * g + t;
-        if (d < a.kv_rank) orow[d] = from_f32<TO>(o[db][t] * inv);
-      }
-    return;
-  }
-  const int64_t slot = ((int64_t)tile * a.splits + split) * 16 + r;
-  float* po = a.part_o + slot * a.kv_rank;
+  l = row_total(l);
+  if (!row_ok) return;
+  if (a.sink) l += sink_weight_log2(a.sink[my_head], m);
+  const float inv = l > 0.f ? 1.0f / l : 0.f;
+  TO* orow = (TO*)a.out + (int64_t)my_row * a.kv_rank;
 #pragma unroll
   for (int db = 0; db < DB; ++db)
 #pragma unroll
-    for (int t = 0; t < 4; ++t) {
-      const int d = 16 * db + 4 * g + t;
-      if (d < a.kv_rank) po[d] = o[db][t];
+    for (int e = 0; e < 4; ++e) {
+      const int d = 16 * db + 4 * g + e;
+      if (d < a.kv_rank) orow[d] = from_f32<TO>(o[db][e] * inv);
     }
-  if (g == 0) {
-    a.part_ml[2 * slot] = m;
-    a.part_ml[2 * slot + 1] = l;
+}
+
+// Few tiles: a workgroup per (tile, share of its keys).  Of every 32 NW keys each of the NW
+// wavefronts stages and scores 32; with the rows' largest scores and the weights exchanged
+// through LDS, each then adds up its share of the columns over all of them.  With one share
+// of the keys the rows are finished here, else the share's results go to the merge kernel.
+template <int KS, int DB, int NW, typename TO>
+__global__ __launch_bounds__(NW* kWave) void latent_attention_split_kernel(LatentMfmaArgs a) {
+  constexpr int PIECES = (4 * KS + 7) / 8, OWN = (DB + NW - 1) / NW;
+  // rows a lane's loads are in flight for at once: as many as registers allow
+  constexpr int ROWS = KS > 10 ? 2 : 4;
+  extern __shared__ __attribute__((aligned(16))) unsigned char lds_raw[];   // [NW][32][stride]
+  __shared__ bf16x8_l p_s[NW][kWave];
+  __shared__ float m_s[NW][16], l_s[NW][16];
+  const int dl = a.kv_rank + a.rot_dim, P = a.page_size;
+  const int stride = dl + kLatentPad;
+  const int wave = threadIdx.x / kWave, lane = threadIdx.x % kWave, r = lane % 16, g = lane / 16;
+  bf16_t* all_s = (bf16_t*)lds_raw;
+  bf16_t* k_s = all_s + wave * 32 * stride;
+  const int tile = blockIdx.x, split = blockIdx.y;
+  const int row0 = a.tiles[3 * tile], nrows = a.tiles[3 * tile + 1];
+  const int* tab = a.table + (int64_t)a.tiles[3 * tile + 2] * a.table_width;
+  const bool row_ok = r < nrows;
+  const int my_row = row0 + max(0, min(r, nrows - 1));
+  const int my_head = my_row % a.heads, my_token = my_row / a.heads;
+  const int pos_r = a.positions[my_token];
+  const int my_pos = row_ok ? pos_r : -1;
+  const int lo_r = a.window > 0 ? max(0, pos_r - a.window + 1) : 0;
+  const int pos_first = a.positions[row0 / a.heads];
+  const int hi_t = a.positions[(row0 + nrows - 1) / a.heads];
+  const int lo_t = a.window > 0 ? max(0, pos_first - a.window + 1) : 0;
+  const int k_begin = (lo_t / 32) * 32 + split * a.keys_per_split;
+  const int k_end = min(k_begin + a.keys_per_split, hi_t + 1);
+  const int64_t slot = ((int64_t)tile * a.splits + split) * 16 + r;
+  if (k_begin >= k_end) {        // more shares than keys: a neutral result, no data touched
+    if (threadIdx.x < 16) {
+      a.part_ml[2 * slot] = -INFINITY;
+      a.part_ml[2 * slot + 1] = 0.f;
+    }
+    return;
   }
+  const int parts = dl / 8, key8 = lane / 8, piece = lane % 8;
+  const float scale_log2 = a.scale * 1.44269504088896341f;
+  bf16x8_l q[KS];
+  f32x4_l o[OWN];
+#pragma unroll
+  for (int db = 0; db < OWN; ++db) o[db] = f32x4_l{0.f, 0.f, 0.f, 0.f};
+  float m = -INFINITY, l = 0.f;            // l: this lane's share of its wavefront's keys
+  for (int kb0 = k_begin; kb0 < k_end; kb0 += 32 * NW) {
+    const int kb = kb0 + 32 * wave;
+#pragma unroll 1
+    for (int c0 = 0; c0 < 4; c0 += ROWS) {
+      int page[ROWS];
+#pragma unroll
+      for (int c = 0; c < ROWS; ++c) {
+        const int j = kb + 8 * (c0 + c) + key8;
+        page[c] = (j >= lo_t && j < k_end) ? tab[j / P] : -1;
+      }
+      bf16x8_l held[ROWS][PIECES];
+#pragma unroll
+      for (int c = 0; c < ROWS; ++c) {
+        const bf16_t* row = a.pages + ((int64_t)max(page[c], 0) * P + (kb + 8 * (c0 + c) + key8) % P) * dl;
+#pragma unroll
+        for (int i = 0; i < PIECES; ++i)
+          held[c][i] = *(const bf16x8_l*)(row + 8 * min(piece + 8 * i, parts - 1));
+      }
+      const bf16x8_l zero = {0, 0, 0, 0, 0, 0, 0, 0};
+#pragma unroll
+      for (int c = 0; c < ROWS; ++c)
+#pragma unroll
+        for (int i = 0; i < PIECES; ++i)
+          if (piece + 8 * i < parts)
+            *(bf16x8_l*)(k_s + (8 * (c0 + c) + key8) * stride + 8 * (piece + 8 * i)) =
+                page[c] >= 0 ? held[c][i] : zero;
+    }
+    if (kb0 == k_begin) load_query_row<KS>(q, a.qa + (int64_t)my_token * a.q_ld + my_head * dl, dl, g);
+    // (a wavefront's LDS accesses are carried out in order: its own rows need no barrier)
+    float sc[8];
+    const float mx = score_block<KS>(sc, q, k_s, stride, kb, dl, scale_log2, my_pos, lo_r, r, g);
+    if (g == 0) m_s[wave][r] = mx;
+    __syncthreads();                       // every wavefront's rows and largest scores are there
+    float m_new = m;
+#pragma unroll
+    for (int w = 0; w < NW; ++w) m_new = fmaxf(m_new, m_s[w][r]);
+    const float m_use = fmaxf(m_new, -1e30f);
+    const float corr = __builtin_amdgcn_exp2f(m - m_use);
+    bf16x8_l pv;
+    l = l * corr + weigh_block(pv, sc, m_use);
+    m = m_new;
+    p_s[wave][lane] = pv;
+    __syncthreads();                       // and every wavefront's weights
+#pragma unroll
+    for (int db = 0; db < OWN; ++db) o[db] = o[db] * corr;
+#pragma unroll 1
+    for (int w = 0; w < NW; ++w)
+      value_block<OWN>(o, p_s[w][lane], all_s + w * 32 * stride, stride, a.kv_rank, wave * OWN, r, g);
+    __syncthreads();                       // before the areas are written again
+  }
+  const float share = row_total(l);
+  if (g == 0) l_s[wave][r] = share;
+  __syncthreads();
+  if (!row_ok) return;
+  float sum = 0.f;
+#pragma unroll
+  for (int w = 0; w < NW; ++w) sum += l_s[w][r];
+  float inv = 1.f;
+  if (a.splits > 1) {
+    if (wave == 0 && g == 0) {
+      a.part_ml[2 * slot] = m;
+      a.part_ml[2 * slot + 1] = sum;
+    }
+  } else {
+    if (a.sink) sum += sink_weight_log2(a.sink[my_head], m);
+    inv = sum > 0.f ? 1.0f / sum : 0.f;
+  }
+#pragma unroll
+  for (int db = 0; db < OWN; ++db)
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      const int d = 16 * (wave * OWN + db) + 4 * g + e;
+      if (d < a.kv_rank) {
+        if (a.splits > 1) a.part_o[slot * a.kv_rank + d] = o[db][e];
+        else ((TO*)a.out)[(int64_t)my_row * a.kv_rank + d] = from_f32<TO>(o[db][e] * inv);
+      }
+    }
 }
 
 // One workgroup per (tile, row): the shares' results weighted by exp(m_s - max m) and
@@ -531,44 +711,73 @@ __global__ __launch_bounds__(128) void latent_attention_merge_kernel(LatentMfmaA
     float total = 0.f;
     for (int s = threadIdx.x; s < a.splits; s += kWave) {
       const float ms = a.part_ml[2 * (base + 16 * s)];
-      const float w = ms == -INFINITY ? 0.f : expf(ms - mx);
+      const float w = ms == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(ms - mx);
       w_s[s] = w;
       total += a.part_ml[2 * (base + 16 * s) + 1] * w;
     }
     total = wave_sum(total);
-    if (a.sink) total += sink_weight(a.sink[(a.tiles[3 * tile] + r) % a.heads], mx);
+    if (a.sink) total += sink_weight_log2(a.sink[(a.tiles[3 * tile] + r) % a.heads], mx);
     if (threadIdx.x == 0) w_s[a.splits] = total > 0.f ? 1.0f / total : 0.f;
   }
   __syncthreads();
   const float inv = w_s[a.splits];
+  // shares beyond the row's keys are empty and wrote no values: what is there is dropped
+  int used = a.splits;
+  while (used > 1 && w_s[used - 1] == 0.f) --used;
   TO* orow = (TO*)a.out + (int64_t)(a.tiles[3 * tile] + r) * a.kv_rank;
   for (int d = threadIdx.x; d < a.kv_rank; d += blockDim.x) {
     float acc = 0.f;
     int s = 0;
-    for (; s + 8 <= a.splits; s += 8) {
+    for (; s + 8 <= used; s += 8) {
       float v[8];
 #pragma unroll
       for (int u = 0; u < 8; ++u) v[u] = a.part_o[(base + 16 * (s + u)) * a.kv_rank + d];
 #pragma unroll
-      for (int u = 0; u < 8; ++u) acc = fmaf(v[u], w_s[s + u], acc);
+      for (int u = 0; u < 8; ++u) acc = w_s[s + u] == 0.f ? acc : fmaf(v[u], w_s[s + u], acc);
     }
-    for (; s < a.splits; ++s) acc = fmaf(a.part_o[(base + 16 * s) * a.kv_rank + d], w_s[s], acc);
+    for (; s < used; ++s)
+      if (w_s[s] != 0.f) acc = fmaf(a.part_o[(base + 16 * s) * a.kv_rank + d], w_s[s], acc);
     orow[d] = from_f32<TO>(acc * inv);
   }
+}
+
+// An LDS size above the default has to be allowed per kernel, once.
+static int allow_lds(const void* kernel, size_t bytes, size_t* allowed) {
+  if (bytes <= *allowed) return 0;
+  if (hipFuncSetAttribute(kernel, hipFuncAttributeMaxDynamicSharedMemorySize, (int)bytes) != hipSuccess)
+    TS_FAIL("latent_attention_mfma: cannot raise the LDS limit to %zu bytes", bytes);
+  *allowed = bytes;
+  return 0;
+}
+
+constexpr size_t kLatentLds = 154 * 1024;      // of a compute unit's 160 KB, beside weights and statistics
+
+template <int KS, int DB, typename TO>
+static int launch_latent_typed(const LatentMfmaArgs& a, int num_tiles, int waves, hipStream_t stream) {
+  const size_t block = (size_t)32 * (a.kv_rank + a.rot_dim + kLatentPad) * sizeof(bf16_t);
+  if (waves == 4) {
+    static size_t allowed = 48 * 1024;         // per instantiation, here and below
+    auto kernel = latent_attention_mfma_kernel<KS, DB, TO>;
+    if (allow_lds((const void*)kernel, 2 * block, &allowed)) return -1;
+    hipLaunchKernelGGL(kernel, dim3(num_tiles / 4), dim3(4 * kWave), 2 * block, stream, a);
+    return 0;
+  }
+  // four wavefronts' rows in LDS at once where a row is short enough, else two's
+  constexpr int NW = (size_t)4 * 32 * (32 * KS + kLatentPad) * sizeof(bf16_t) <= kLatentLds ? 4 : 2;
+  static size_t allowed = 48 * 1024;
+  auto kernel = latent_attention_split_kernel<KS, DB, NW, TO>;
+  if (allow_lds((const void*)kernel, NW * block, &allowed)) return -1;
+  hipLaunchKernelGGL(kernel, dim3(num_tiles, a.splits), dim3(NW * kWave), NW * block, stream, a);
+  if (a.splits > 1)
+    hipLaunchKernelGGL(latent_attention_merge_kernel<TO>, dim3(num_tiles, 16), dim3(128),
+                       (size_t)(a.splits + 1) * sizeof(float), stream, a);
+  return 0;
 }
 
 template <int KS, int DB>
 static int launch_latent_mfma(const LatentMfmaArgs& a, int num_tiles, int waves, int out_type,
                               hipStream_t stream) {
-  const int dl = a.kv_rank + a.rot_dim;
-  const size_t lds = (size_t)32 * (dl + kLatentPad) * sizeof(bf16_t) + 32 * sizeof(int);
-  TS_DISPATCH_TYPE(out_type, TO, {
-    hipLaunchKernelGGL((latent_attention_mfma_kernel<KS, DB, TO>),
-                       dim3(num_tiles / waves, a.splits), dim3(waves * kWave), lds, stream, a);
-    if (a.splits > 1)
-      hipLaunchKernelGGL(latent_attention_merge_kernel<TO>, dim3(num_tiles, 16), dim3(128),
-                         (size_t)(a.splits + 1) * sizeof(float), stream, a);
-  });
+  TS_DISPATCH_TYPE(out_type, TO, return (launch_latent_typed<KS, DB, TO>(a, num_tiles, waves, stream)));
   return 0;
 }
 
@@ -578,8 +787,9 @@ extern "C" int ts_latent_attention_mfma_fits(int kv_rank, int rot_dim) {
   return dl % 8 == 0 && dl <= 640 && kv_rank <= 512;
 }
 
-// `tiles` comes in groups of `waves` (1 or 4) tiles of one entry, a group's last tiles
-// possibly empty (0 rows); `num_tiles` counts them all.
+// `waves` 4: `tiles` comes in groups of four tiles of one entry, a group's last tiles possibly
+// empty (0 rows), `num_tiles` counts them all and keys are not shared out; 1: every tile has
+// rows and its keys are shared out in `splits` runs.
 extern "C" int ts_latent_attention_mfma(const float* qa, const void* pages, void* out,
                                         int out_type, const int* tiles, int num_tiles, int waves,
                                         const int* positions, const int* table, int table_width,
@@ -594,16 +804,19 @@ extern "C" int ts_latent_attention_mfma(const float* qa, const void* pages, void
   if (splits < 1 || keys_per_split < 32 || keys_per_split % 32)
     TS_FAIL("latent_attention_mfma: bad split of the keys (%d runs of %d)", splits, keys_per_split);
   if (splits > 1 && (!part_o || !part_ml)) TS_FAIL("latent_attention_mfma: no scratch for the shares");
-  if ((waves != 1 && waves != 4) || num_tiles % waves)
+  if ((waves != 1 && waves != 4) || num_tiles % waves || (waves == 4 && splits != 1))
     TS_FAIL("latent_attention_mfma: %d tiles in groups of %d", num_tiles, waves);
-  if (((uintptr_t)pages & 15) != 0) TS_FAIL("latent_attention_mfma: pages must start on 16 bytes");
+  if ((((uintptr_t)pages | (uintptr_t)qa) & 15) != 0 || q_ld % 4)
+    TS_FAIL("latent_attention_mfma: pages and query rows must start on 16 bytes");
   LatentMfmaArgs a{qa, (const bf16_t*)pages, out, tiles, positions, table, part_o, part_ml,
                    table_width, page_size, heads, kv_rank, rot_dim, window, keys_per_split, splits,
                    scale, q_ld, sink};
   const int dl = kv_rank + rot_dim;
   int rc;
   if (dl <= 96 && kv_rank <= 64) rc = launch_latent_mfma<3, 4>(a, num_tiles, waves, out_type, stream);
+  else if (dl <= 160 && kv_rank <= 128) rc = launch_latent_mfma<5, 8>(a, num_tiles, waves, out_type, stream);
   else if (dl <= 320 && kv_rank <= 256) rc = launch_latent_mfma<10, 16>(a, num_tiles, waves, out_type, stream);
+  else if (dl <= 576) rc = launch_latent_mfma<18, 32>(a, num_tiles, waves, out_type, stream);
   else rc = launch_latent_mfma<20, 32>(a, num_tiles, waves, out_type, stream);
   if (rc) return rc;
   TS_CHECK_LAUNCH("latent_attention_mfma");

@@ -1656,21 +1656,25 @@ class HipOps:
         over several wavefronts and merged."""
         d = self.dispatch
         counts = [-(-n * heads // 16) for n in batch.q_lens]
-        # many tiles: four of one entry to a workgroup, which walk their keys together; few:
-        # one tile a workgroup (and three empty ones), every tile's keys shared out
+        # many tiles: four of one entry to a workgroup, which walk their keys together, the
+        # longest walks first (a compute unit holds one such workgroup at a time); few: one
+        # tile a workgroup, every tile's keys shared out over its wavefronts and over workgroups
         waves = 1 if sum(counts) < d.latent_full_tiles else 4
         key = ("latent_tiles", heads, waves)
         if key not in batch.plans:
-            tiles, row = [], 0
-            for e, n in enumerate(batch.q_lens):
+            lists, keys, row = [], [], 0
+            for e, (n, start) in enumerate(zip(batch.q_lens, batch.starts)):
                 rows = n * heads
-                for i in range(0, rows, 16):
-                    tiles.append((row + i, min(16, rows - i), e))
-                    while waves == 1 and len(tiles) % 4:
-                        tiles.append((row, 0, e))       # empty tiles fill the workgroup
-                while len(tiles) % 4:
-                    tiles.append((row, 0, e))
+                firsts = np.arange(0, -(-rows // (16 * waves)) * 16 * waves, 16)
+                there = np.clip(rows - firsts, 0, 16)
+                lists.append(np.stack([row + np.where(there > 0, firsts, 0), there,
+                                       np.full_like(firsts, e)], axis=1))
+                keys.append(start + np.minimum(firsts[::waves] // heads + -(-16 * waves // heads), n))
                 row += rows
+            tiles = np.concatenate(lists)
+            if waves == 4:
+                order = np.argsort(-np.concatenate(keys), kind="stable")
+                tiles = tiles.reshape(-1, 4, 3)[order].reshape(-1, 3)
             batch.plans[key] = (self._upload_ints(tiles), len(tiles))
         tiles, num_tiles = batch.plans[key]
         # the longest run of keys a workgroup can have: the window and its own tokens, or
@@ -1680,8 +1684,9 @@ class HipOps:
         # up to 31 keys more than the span have to be covered
         splits, per = 1, 1 << 30
         if waves == 1:
-            most = max(1, d.latent_full_tiles // (num_tiles // 4))
-            per = -(-max(d.latent_split_keys, -(-(span + 31) // most)) // 32) * 32
+            most = max(1, d.latent_workgroups // num_tiles)
+            run = d.latent_split_keys
+            per = max(1, -(-(span + 31) // (most * run))) * run
             splits = -(-(span + 31) // per)
             if splits == 1:
                 per = 1 << 30
@@ -1692,7 +1697,7 @@ class HipOps:
             part_ml = torch.empty(num_tiles, splits, 16, 2, dtype=torch.float32,
                                   device=self.device)
         self._call(self.lib.ts_latent_attention_mfma, _ptr(qa), _ptr(cache.k_pages), _ptr(out),
-                   _TYPE_CODE[out.dtype], _ptr(tiles), num_tiles, 4, _ptr(batch.positions),
+                   _TYPE_CODE[out.dtype], _ptr(tiles), num_tiles, waves, _ptr(batch.positions),
                    _ptr(table), table.shape[1], cache.page_size, heads, kv_rank, rot_dim,
                    int(window) if window else 0, c_float(scale), per, splits, _ptr(part_o),
                    _ptr(part_ml), q_ld, _ptr(sink), self._stream())
