@@ -631,14 +631,14 @@ def test_greedy_generation_in_bfloat16_through_captured_graphs(gpu_device, tmp_p
 def test_sizes_that_are_multiples_of_nothing(gpu_device, tmp_path, dtype):
     """Odd head sizes, a width and inner sizes that are multiples of no tile or vector width:
     the products fall to the multiply-add kernels and heads are padded."""
-    cfg = fubepel_config(width=34, vocab=61, eps=1e-6, embed_scale=1.7, side_dim=5, layers=[
+    cfg = fubepel_config(width=34, vocab=61, eps=1e-6, embed_scale=1.7, side_dim=13, layers=[
         fubepel_latent(heads=3, dim=5, rot_dim=6, vdim=7, kv_rank=13, scale=0.1, base=800.0,
-                       mlp=fubepel_dense(9, 0.9)),
-        fubepel_delta(heads=3, kv_heads=1, dim=7, vdim=5, conv=2, mlp=None),
-        fubepel_attention(heads=1, kv_heads=1, dim=6, vdim=10, scale=0.3, window=11, keep_first=3,
-                          mlp=fubepel_dense(5, 2.0)),
-        fubepel_latent(heads=2, dim=3, rot_dim=6, vdim=1, kv_rank=13, scale=0.1, base=800.0, kv_from=0,
-                       mlp=fubepel_dense(3, 1.0))])
+                       mlp=fubepel_dense(29, 0.9)),
+        fubepel_delta(heads=3, kv_heads=1, dim=7, vdim=11, conv=2, mlp=None),
+        fubepel_attention(heads=3, kv_heads=3, dim=6, vdim=10, scale=0.3, window=11, keep_first=3,
+                          mlp=fubepel_dense(35, 2.0)),
+        fubepel_latent(heads=2, dim=3, rot_dim=6, vdim=9, kv_rank=13, scale=0.1, base=800.0, kv_from=0,
+                       mlp=fubepel_dense(23, 1.0))])
     d = write_fubepel_model(tmp_path, cfg, 12, dtype, sharpen=1.0)
     pcfg, w = plain.read_model_dir(d)
     _, model = load_model(d, dtype, gpu_device)
