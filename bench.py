@@ -605,8 +605,8 @@ def compare_designs(args) -> int:
             _, engine = make_engine(raw, args.dtype, None, b, max_len, 4096, page, model=model)
             sec, decoded, held = decode_run(engine, b, ctx - 128, steps, warmup, vocab, max_tokens)
             del engine
-            params = sum(t.numel() for part in model.parts() for t in part.held_tensors()
-                         if t.dim() == 2)
+            params = sum({t.data_ptr(): t.numel() for part in model.parts()
+                          for t in part.held_tensors() if t.dim() == 2}.values())
             row[kind] = {
                 "matrix_params_m": round(params / 1e6, 1),
                 "prefill_tok_s": round(T / pre, 1), "prefill_ms": round(pre * 1e3, 3),

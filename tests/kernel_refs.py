@@ -233,6 +233,9 @@ class TorchOps:
         gate = 0.5 * z * (1.0 + torch.tanh(0.7978845608028654 * (z + 0.044715 * z ** 3)))
         return (gate * table[ids.long(), col:col + z.shape[1]].float()).to(out_dtype)
 
+    def token_gate_linear(self, z, table, ids, col, weight, act_dtype):
+        return self.linear(self.token_gate(z, table, ids, col, act_dtype), weight, torch.float32)
+
     def postnorm_add_norm(self, resid, delta, post_w, post_eps, norm_w, norm_eps, out_dtype):
         self.postnorm_add(resid, delta, post_w, post_eps)
         return (self._unit(resid, norm_eps) * norm_w.float()).to(out_dtype)

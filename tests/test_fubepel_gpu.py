@@ -74,6 +74,18 @@ def test_gate_of_a_tokens_own_row(gpu_device):
                 close(ops.token_gate(z, table, ids, index * dim, out_dtype),
                       REF.token_gate(z, table, ids, index * dim, out_dtype),
                       **(dict(rtol=1e-5, atol=1e-5) if out_dtype == torch.float32 else dict(rtol=1e-2, atol=1e-2)))
+    # with the product behind it: one kernel for few rows of bfloat16, two for the others
+    for T, dim, parts, index, width in ((1, 16, 3, 1, 40), (8, 128, 8, 7, 2048), (17, 24, 2, 0, 70), (64, 8, 1, 0, 64),
+                                        (65, 16, 2, 1, 48), (5, 6, 2, 1, 33), (40, 512, 1, 0, 100), (3, 520, 1, 0, 16)):
+        for dtype in (torch.float32, torch.bfloat16):
+            z = rnd((T, dim), 1, 3.0).to(gpu_device)
+            table = rnd((30, parts * dim), 2).to(dtype).to(gpu_device)
+            w = rnd((width, dim), 5, dim ** -0.5).to(dtype).to(gpu_device)
+            ids = torch.randint(0, 30, (T,), generator=torch.Generator().manual_seed(3)).int().to(gpu_device)
+            got = ops.token_gate_linear(z, table, ids, index * dim, w, dtype)
+            assert got.dtype == torch.float32
+            close(got, REF.token_gate_linear(z, table, ids, index * dim, w, dtype),
+                  **(dict(rtol=1e-4, atol=1e-4) if dtype == torch.float32 else dict(rtol=1e-2, atol=1e-2)))
     with pytest.raises(ValueError, match="columns"):
         ops.token_gate(torch.zeros(2, 8, device=gpu_device), torch.zeros(4, 12, device=gpu_device),
                        torch.zeros(2, dtype=torch.int32, device=gpu_device), 8, torch.float32)

@@ -109,15 +109,19 @@ __global__ __launch_bounds__(1024) void postnorm_add_kernel(
   float* x = resid + row * width;
   const TD* d = delta + row * width;
   TO* o = out + row * width;
-  float dc[kRowItems], xc[kRowItems];
+  // (the weights are asked for with the row, not behind the sum that they wait for)
+  float dc[kRowItems], xc[kRowItems], pc[kRowItems], nc[kRowItems];
   float ss = 0.f;
 #pragma unroll
   for (int k = 0; k < kRowItems; ++k) {
     const int i = threadIdx.x + k * nt;
     dc[k] = i < width ? to_f32(d[i]) : 0.f;
     xc[k] = i < width ? x[i] : 0.f;
-    ss += dc[k] * dc[k];
+    pc[k] = i < width ? post_w[i] : 0.f;
+    nc[k] = THEN == kThenNorm && i < width ? norm_w[i] : 0.f;
   }
+#pragma unroll
+  for (int k = 0; k < kRowItems; ++k) ss += dc[k] * dc[k];
   for (int i = threadIdx.x + kRowItems * nt; i < width; i += nt) {
     const float v = to_f32(d[i]);
     ss += v * v;
@@ -128,7 +132,7 @@ __global__ __launch_bounds__(1024) void postnorm_add_kernel(
   for (int k = 0; k < kRowItems; ++k) {
     const int i = threadIdx.x + k * nt;
     if (i < width) {
-      xc[k] = xc[k] + dc[k] * r * post_w[i];
+      xc[k] = xc[k] + dc[k] * r * pc[k];
       x[i] = xc[k];
       if (THEN == kThenRows) o[i] = from_f32<TO>(xc[k]);
       ss2 += xc[k] * xc[k];
@@ -145,7 +149,7 @@ __global__ __launch_bounds__(1024) void postnorm_add_kernel(
 #pragma unroll
     for (int k = 0; k < kRowItems; ++k) {
       const int i = threadIdx.x + k * nt;
-      if (i < width) o[i] = from_f32<TO>(xc[k] * r2 * norm_w[i]);
+      if (i < width) o[i] = from_f32<TO>(xc[k] * r2 * nc[k]);
     }
     // each thread reads back the elements it wrote itself
     for (int i = threadIdx.x + kRowItems * nt; i < width; i += nt)
@@ -212,6 +216,98 @@ extern "C" int ts_token_gate(const float* z, const void* table, int table_type, 
                          dim3(256), 0, stream, z, (const TW*)table, ids, (TO*)out, total, dim, ld,
                          col)));
   TS_CHECK_LAUNCH("token_gate");
+  return 0;
+}
+
+// The same gate inside the product that leads back to the stream, for few rows (bfloat16
+// table and weight, bfloat16 gated values as the kernel above writes them):
+// out[t, n] = sum_j (gelu_tanh(z[t, j]) * table[ids[t], col + j]) w[n, j], float32.
+// A workgroup makes the gated values of 16 tokens in LDS and each of its wavefronts owns 16
+// columns of the result.
+typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8_side;
+typedef __attribute__((ext_vector_type(4))) float f32x4_side;
+constexpr int kSideDim = 512;
+
+__global__ __launch_bounds__(256) void token_gate_product_kernel(
+    const float* __restrict__ z, const bf16_t* __restrict__ table, const int* __restrict__ ids,
+    const bf16_t* __restrict__ w, float* __restrict__ out, int num_tokens, int width, int dim,
+    int ld, int col) {
+  extern __shared__ __attribute__((aligned(16))) unsigned char lds_raw[];
+  bf16_t* act = (bf16_t*)lds_raw;                  // [16][stride]
+  const int stride = (dim + 31) / 32 * 32 + 8;
+  const int t0 = blockIdx.y * 16;
+  const int wave = threadIdx.x / kWave, lane = threadIdx.x % kWave, r = lane % 16, g = lane / 16;
+  const int n0 = (blockIdx.x * 4 + wave) * 16, n = min(n0 + r, width - 1);
+  const bf16x8_side zero = {0, 0, 0, 0, 0, 0, 0, 0};
+  // The first four steps' weights are asked for before the gated values' chain of loads (a
+  // token's id, then its row of the table) begins.
+  constexpr int kEarly = 4;
+  bf16x8_side early[kEarly];
+#pragma unroll
+  for (int i = 0; i < kEarly; ++i)
+    early[i] = *(const bf16x8_side*)(w + (int64_t)n * dim + min(32 * i + 8 * g, dim - 8));
+  const bool wide = ld % 8 == 0 && col % 8 == 0 && ((uintptr_t)table & 15) == 0;
+  const int units = (stride - 8) / 8;              // runs of eight values a token, padding included
+  for (int u = threadIdx.x; u < 16 * units; u += blockDim.x) {
+    const int row = u / units, j0 = (u - row * units) * 8;
+    const int t = min(t0 + row, num_tokens - 1);
+    bf16x8_side v = zero;
+    if (t0 + row < num_tokens && j0 < dim) {
+      const float* zr = z + (int64_t)t * dim + j0;
+      const bf16_t* er = table + (int64_t)ids[t] * ld + col + j0;
+      bf16x8_side e;
+      if (wide) {
+        e = *(const bf16x8_side*)er;
+      } else {
+#pragma unroll
+        for (int j = 0; j < 8; ++j) e[j] = er[j];
+      }
+      const f32x4_side a = *(const f32x4_side*)zr, b = *(const f32x4_side*)(zr + 4);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) v[j] = (bf16_t)(gelu_tanh(j < 4 ? a[j] : b[j - 4]) * (float)e[j]);
+    }
+    *(bf16x8_side*)(act + row * stride + j0) = v;
+  }
+  __syncthreads();
+  f32x4_side acc = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+  for (int i = 0; i < kEarly; ++i) {
+    if (32 * i < dim) {            // (past the last column the gated values are zeros)
+      const bf16x8_side av = *(const bf16x8_side*)(act + r * stride + 32 * i + 8 * g);
+      acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(early[i], av, acc, 0, 0, 0);
+    }
+  }
+  for (int k = 32 * kEarly; k < dim; k += 32) {
+    const int at = k + 8 * g;
+    const bf16x8_side wv = *(const bf16x8_side*)(w + (int64_t)n * dim + min(at, dim - 8));
+    const bf16x8_side av = *(const bf16x8_side*)(act + r * stride + at);
+    acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wv, av, acc, 0, 0, 0);
+  }
+  // lane (r, g) holds columns n0 + 4 g .. + 3 of token r
+  if (t0 + r >= num_tokens) return;
+  float* o = out + (int64_t)(t0 + r) * width + n0 + 4 * g;
+#pragma unroll
+  for (int e = 0; e < 4; ++e)
+    if (n0 + 4 * g + e < width) o[e] = acc[e];
+}
+
+extern "C" int ts_token_gate_product_fits(int num_tokens, int dim) {
+  return num_tokens <= 64 && dim % 8 == 0 && dim <= kSideDim;
+}
+
+extern "C" int ts_token_gate_product(const float* z, const void* table, const int* ids,
+                                     const void* w, float* out, int num_tokens, int width,
+                                     int dim, int ld, int col, hipStream_t stream) {
+  if (num_tokens <= 0) return 0;
+  if (width <= 0 || dim <= 0 || !ts_token_gate_product_fits(num_tokens, dim))
+    TS_FAIL("token_gate_product: %d tokens of %d values are not taken", num_tokens, dim);
+  if (col < 0 || col + dim > ld) TS_FAIL("token_gate_product: columns [%d, %d) of rows of %d", col, col + dim, ld);
+  if (((uintptr_t)w | (uintptr_t)z) & 15) TS_FAIL("token_gate_product: weight and values must start on 16 bytes");
+  const size_t lds = (size_t)16 * ((dim + 31) / 32 * 32 + 8) * sizeof(bf16_t);
+  hipLaunchKernelGGL(token_gate_product_kernel, dim3((width + 63) / 64, (num_tokens + 15) / 16),
+                     dim3(256), lds, stream, z, (const bf16_t*)table, ids, (const bf16_t*)w, out,
+                     num_tokens, width, dim, ld, col);
+  TS_CHECK_LAUNCH("token_gate_product");
   return 0;
 }
 

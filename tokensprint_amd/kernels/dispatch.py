@@ -91,7 +91,7 @@ class Dispatch:
     # keys (a block of 32 for each wavefront) over up to about `latent_workgroups` workgroups.
     latent_full_tiles: int = 1024
     latent_split_keys: int = 128
-    latent_workgroups: int = 1024
+    latent_workgroups: int = 512
 
 
 #: what each table was measured on -> the table

@@ -1164,6 +1164,24 @@ class HipOps:
                    self._stream())
         return out
 
+    def token_gate_linear(self, z, table, ids, col, weight, act_dtype):
+        """`token_gate` in `act_dtype` times weight [N, dim] transposed -> float32 [T, N]; one
+        kernel for few rows of bfloat16."""
+        T, dim = z.shape
+        if act_dtype == table.dtype == weight.dtype == torch.bfloat16 and \
+                self.lib.ts_token_gate_product_fits(T, dim) == 1:
+            self._check("z", z, torch.float32, ndim=2)
+            self._check("token table", table, torch.bfloat16, ndim=2)
+            self._check("token ids", ids, torch.int32, shape=(T,))
+            self._check("weight", weight, torch.bfloat16, shape=(weight.shape[0], dim))
+            if col < 0 or col + dim > table.shape[1]:
+                raise ValueError(f"token_gate: columns [{col}, {col + dim}) of rows of {table.shape[1]}")
+            out = torch.empty(T, weight.shape[0], dtype=torch.float32, device=self.device)
+            self._call(self.lib.ts_token_gate_product, _ptr(z), _ptr(table), _ptr(ids), _ptr(weight),
+                       _ptr(out), T, weight.shape[0], dim, table.shape[1], int(col), self._stream())
+            return out
+        return self.linear(self.token_gate(z, table, ids, col, act_dtype), weight, torch.float32)
+
     # ------------------------------------------------------------ state-space mixer
     def conv_silu(self, proj, col, channels, weight, bias, batch, state, in_bias=None,
                   plain=False):

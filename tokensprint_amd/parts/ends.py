@@ -124,9 +124,8 @@ class GatedTokenTable(TokenSide):
 
     def forward(self, h, batch):
         z = self.ops.linear(h, self.w_gate, torch.float32)
-        act = self.ops.token_gate(z, self.table, batch.token_ids, self.index * self.dim,
-                                  self.ctx.dtype)
-        return self.ops.linear(act, self.w_proj, torch.float32)
+        return self.ops.token_gate_linear(z, self.table, batch.token_ids, self.index * self.dim,
+                                          self.w_proj, self.ctx.dtype)
 
 
 @register(HEADS, "head")
