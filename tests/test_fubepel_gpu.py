@@ -465,7 +465,7 @@ TOL = (2e-4, 1e-4)
 
 
 def rms_errors(got, want):
-    """Every row's error as replayed traces are judged: root mean square over the vocabulary,
+    """Every row's error: the root mean square of the difference over the vocabulary,
     the mean taken off, in units of the logits' own spread."""
     diff = got - want
     diff = diff - diff.mean(dim=1, keepdim=True)

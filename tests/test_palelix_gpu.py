@@ -428,7 +428,7 @@ def compare(col, ref, rtol, atol):
         got, positions = col.stacked(rid)
         assert positions == list(range(want.shape[0]))
         assert torch.isfinite(got).all()
-        # a row's error as the replayed traces are judged: the root mean square of the
+        # a row's error: the root mean square of the
         # difference over the vocabulary, its mean taken off, in units of the logits' own
         diff = got - want
         diff = diff - diff.mean(dim=1, keepdim=True)
