@@ -67,15 +67,18 @@ class TorchOps:
             else self.linear(h, weight, out_dtype)
         return out, resid
 
-    def linear_silu_mul(self, x, weight, out_dtype, limit=None):
-        return self.silu_mul(self.linear(x, weight, out_dtype), limit)
+    def linear_silu_mul(self, x, weight, out_dtype, limit=None, act="silu"):
+        return self.silu_mul(self.linear(x, weight, out_dtype), limit, act)
 
-    def silu_mul(self, gate_up, limit=None):
+    def silu_mul(self, gate_up, limit=None, act="silu"):
         inner = gate_up.shape[-1] // 2
         g, u = gate_up[:, :inner].float(), gate_up[:, inner:].float()
         if limit is not None:
             g, u = torch.clamp(g, max=limit), torch.clamp(u, -limit, limit)
             return (g * torch.sigmoid(1.702 * g) * (u + 1.0)).to(gate_up.dtype)
+        if act == "gelu_tanh":
+            inside = 0.7978845608028654 * (g + 0.044715 * g ** 3)
+            return (0.5 * g * (1.0 + torch.tanh(inside)) * u).to(gate_up.dtype)
         return (g * torch.sigmoid(g) * u).to(gate_up.dtype)
 
     # ---------------------------------------------------------------- q/k preparation
@@ -240,6 +243,16 @@ class TorchOps:
         self.postnorm_add(resid, delta, post_w, post_eps)
         return (self._unit(resid, norm_eps) * norm_w.float()).to(out_dtype)
 
+    def normed_pair(self, pair, out_dtype):
+        return (self._unit(pair.a.float(), pair.eps) * pair.weight_a.float()
+                + self._unit(pair.b.float(), pair.eps) * pair.weight_b.float()).to(out_dtype)
+
+    def pair_postnorm_add(self, resid, pair, post_w, post_eps, norm_w, norm_eps, out_dtype):
+        self.postnorm_add(resid, self.normed_pair(pair, torch.float32), post_w, post_eps)
+        if norm_w is not None:
+            return (self._unit(resid, norm_eps) * norm_w.float()).to(out_dtype)
+        return self.stream_rows(resid, out_dtype) if out_dtype is not None else None
+
     def norm_token_shift(self, resid, norm_w, eps, shift_w, batch, state, out_dtype):
         h = self._unit(resid.float(), eps) * norm_w.float()
         prev = torch.zeros_like(h)
@@ -296,7 +309,7 @@ class TorchOps:
 
     def linear_recurrence(self, x, q_col, k_col, v_col, batch, state, *, heads, kv_heads, dim,
                           vdim, silu_inputs, decay=None, gates=None, per_channel=False,
-                          delta=False):
+                          delta=False, turn=None, k_scale=1.0):
         T = x.shape[0]
         rep = heads // kv_heads
 
@@ -309,6 +322,15 @@ class TorchOps:
         q = part(q_col, kv_heads, dim).repeat_interleave(rep, dim=1)
         k = part(k_col, kv_heads, dim).repeat_interleave(rep, dim=1)
         v = part(v_col, heads, vdim)
+        if turn is not None:
+            pairs = turn.shape[1]
+            cos, sin = (turn[batch.positions.long()][:, None, :, i] for i in (0, 1))
+
+            def turned(u):
+                a, b = u[..., 0:2 * pairs:2], u[..., 1:2 * pairs:2]
+                both = torch.stack([a * cos - b * sin, b * cos + a * sin], dim=-1).flatten(-2)
+                return torch.cat([both, u[..., 2 * pairs:]], dim=-1)
+            q, k = turned(q), turned(k) * k_scale
         out = torch.empty(T, heads, vdim, dtype=torch.float32, device=x.device)
         for b, lo, hi, slot, start in self._entries(batch):
             S = state[slot].clone() if start > 0 else torch.zeros_like(state[slot])
@@ -334,16 +356,19 @@ class TorchOps:
         width = inner // groups
         yf = y.float().view(T, groups, width)
         yf = yf * torch.rsqrt(yf.pow(2).mean(-1, keepdim=True) + eps)
-        w = norm_w.float()
-        yf = yf * (w.view(1, 1, width) if w.numel() == width else w.view(1, groups, width))
+        if norm_w is not None:
+            w = norm_w.float()
+            yf = yf * (w.view(1, 1, width) if w.numel() == width else w.view(1, groups, width))
         z = gate_rows[:, gate_col:gate_col + inner].float()
         act = torch.sigmoid(z) if gate == "sigmoid" else z * torch.sigmoid(z)
         return (yf.view(T, inner) * act).to(out_dtype)
 
     # ---------------------------------------------------------------- routed experts
     def route_experts(self, logits, *, top, group_count=1, group_keep=1, scores="softmax",
-                      normalize=True, correction=None, weight_scale=1.0):
+                      normalize=True, correction=None, weight_scale=1.0, bias=None):
         T, E = logits.shape
+        if bias is not None:
+            logits = logits.float() + bias.float()
         # sigmoid scores keep the logits' order: experts are ranked by the logits themselves
         rank = logits.float()
         if scores == "softmax":

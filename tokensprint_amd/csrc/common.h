@@ -63,16 +63,22 @@ __device__ __forceinline__ float block_sum(float v, float* scratch) {
   return total;
 }
 
+// 0.5 z (1 + tanh(sqrt(2 / pi) (z + 0.044715 z^3))), the tanh form of GELU.
+__device__ __forceinline__ float gelu_tanh(float z) {
+  return 0.5f * z * (1.0f + tanhf(0.79788456080286536f * (z + 0.044715f * z * z * z)));
+}
+
 // A gated feed-forward's unit, from the results of its two products (rounded to the
 // activation type first wherever a product makes it in its epilogue, as the path through
 // memory stores them): silu(gate) * up, or, with a
 // positive limit, g sigmoid(1.702 g) (u + 1) of g = min(gate, limit) and u = up held
-// between -limit and limit.
+// between -limit and limit, or, with a negative limit, gelu_tanh(gate) * up.
 __device__ __forceinline__ float gated_unit(float gate, float up, float limit) {
   if (limit > 0.f) {
     const float g = fminf(gate, limit), u = fminf(fmaxf(up, -limit), limit);
     return g / (1.f + expf(-1.702f * g)) * (u + 1.f);
   }
+  if (limit < 0.f) return gelu_tanh(gate) * up;
   return gate / (1.f + expf(-gate)) * up;
 }
 

@@ -12,11 +12,11 @@
 // large logits' sigmoids round to the same number).  `normalize` 0: the weights are the
 // chosen experts' scores as they are.  `correction` (float32 [E] or null): groups and experts
 // are ranked by score + correction, the weights stay the scores.  `weight_scale`: a factor on
-// the weights.
+// the weights.  `bias` (float32 [E] or null) is added to the logits first.
 __global__ __launch_bounds__(256) void route_experts_kernel(
     const float* __restrict__ logits, float* __restrict__ weights, int rows, int E, int top,
     int group_count, int group_keep, int sigmoid_scores, int normalize,
-    const float* __restrict__ correction, float weight_scale) {
+    const float* __restrict__ correction, float weight_scale, const float* __restrict__ bias) {
   extern __shared__ float lds[];
   const int wave = threadIdx.x / kWave, lane = threadIdx.x % kWave;
   const int64_t t = (int64_t)blockIdx.x * (blockDim.x / kWave) + wave;
@@ -25,20 +25,21 @@ __global__ __launch_bounds__(256) void route_experts_kernel(
   float* open = score + E;                       // the rank while the expert can be chosen, else -inf
   float* taken = open + E;                       // 1 for a chosen expert
   float* best = taken + E;                       // [group_count]
-  const float* z = logits + (live ? t : 0) * E;
+  const float* zr = logits + (live ? t : 0) * E;
+  auto z = [&](int e) { return bias ? zr[e] + bias[e] : zr[e]; };
   const int per = E / group_count;
   if (sigmoid_scores) {
     for (int e = lane; e < E; e += kWave) {
-      score[e] = 1.0f / (1.0f + expf(-z[e]));
-      open[e] = z[e];
+      score[e] = 1.0f / (1.0f + expf(-z(e)));
+      open[e] = z(e);
     }
   } else {
     float m = -INFINITY;
-    for (int e = lane; e < E; e += kWave) m = fmaxf(m, z[e]);
+    for (int e = lane; e < E; e += kWave) m = fmaxf(m, z(e));
     m = wave_max(m);
     float sum = 0.f;
     for (int e = lane; e < E; e += kWave) {
-      const float p = expf(z[e] - m);
+      const float p = expf(z(e) - m);
       score[e] = p;
       sum += p;
     }
@@ -92,7 +93,7 @@ __global__ __launch_bounds__(256) void route_experts_kernel(
 extern "C" int ts_route_experts(const float* logits, float* weights, int rows, int experts,
                                 int top, int group_count, int group_keep, int sigmoid_scores,
                                 int normalize, const float* correction, float weight_scale,
-                                hipStream_t stream) {
+                                const float* bias, hipStream_t stream) {
   if (rows <= 0) return 0;
   if (experts <= 0 || group_count <= 0 || experts % group_count || group_keep <= 0 ||
       group_keep > group_count || top <= 0 || top > group_keep * (experts / group_count))
@@ -103,7 +104,7 @@ extern "C" int ts_route_experts(const float* logits, float* weights, int rows, i
   if (correction && sigmoid_scores) TS_FAIL("route_experts: a correction goes with softmax scores");
   hipLaunchKernelGGL(route_experts_kernel, dim3((rows + 3) / 4), dim3(256), lds, stream, logits,
                      weights, rows, experts, top, group_count, group_keep, sigmoid_scores, normalize,
-                     correction, weight_scale);
+                     correction, weight_scale, bias);
   TS_CHECK_LAUNCH("route_experts");
   return 0;
 }

@@ -63,7 +63,7 @@ struct DirectArgs {
   const float* merge_ml;    // [items, merge_splits, 16, 2]: row maximum (log2 units), sum
   const int* merge_pos;     // [M]: position of each row's token
   int merge_splits, merge_nkv, merge_group, merge_hd, merge_window, merge_chunk;
-  float limit;              // pair: gated_unit's limit (0: silu)
+  float limit;              // pair: gated_unit's limit (0: silu, below: gelu)
 };
 
 // Launches it; `norm` (the fused form) takes at most 16 rows.  Returns 0 or -1 with the

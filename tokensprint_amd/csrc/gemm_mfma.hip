@@ -133,7 +133,7 @@ struct StagedArgs {
   int kc;                   // K elements staged per round (multiple of WK*128, or >= K)
   int rstd_offset;          // byte offset in LDS of the fused form's row factors
   float eps;
-  float limit;              // PAIR: gated_unit's limit (0: silu)
+  float limit;              // PAIR: gated_unit's limit (0: silu, below: gelu)
 };
 
 template <int MT, int WN, int WK, typename TC, bool PAIR, bool NORM>
@@ -369,7 +369,7 @@ static int dispatch_skinny(const void* a, const void* w, void* c, int M, int N, 
 }
 
 // pair = 1: W is [2, N, K] (gate rows then up rows) and C[M, N] = silu(A Wg^T) * (A Wu^T), or,
-// with a limit above 0, gated_unit's other form.
+// with a limit other than 0, gated_unit's other forms.
 extern "C" int ts_gemm_mfma_bf16(const void* a, const void* w, void* c, int c_type, int M,
                                  int N, int K, int pair, float limit, hipStream_t stream) {
   if (M <= 0 || N <= 0) return 0;

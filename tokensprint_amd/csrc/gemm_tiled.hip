@@ -10,7 +10,7 @@ extern "C" int ts_gemm_tiled_fits(int M, int N, int K, int pair) {
 }
 
 // C[M, N] = A[M, K] W[N, K]^T, or with `pair` C[M, N] = silu(A Wg^T) * (A Wu^T) (or, with a
-// `limit`, gated_unit's other form) for W = [Wg; Wu] of 2 N rows.  `c_type`: bfloat16 or float32 (float32 not with `pair`).
+// `limit` other than 0, gated_unit's other forms) for W = [Wg; Wu] of 2 N rows.  `c_type`: bfloat16 or float32 (float32 not with `pair`).
 // `tile`: 0 lets the sizes choose; 1 to 5 name a tile (for measuring; the result is the
 // same to the bit).
 extern "C" int ts_gemm_tiled_bf16(const void* a, const void* w, void* c, int c_type, int M, int N,

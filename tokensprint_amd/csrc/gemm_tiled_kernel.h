@@ -58,7 +58,7 @@ struct TiledArgs {
   const float* norm_w;
   bf16_t* prepared;
   float* sumsq_out;
-  float limit;          // PAIR: gated_unit's limit (0: silu)
+  float limit;          // PAIR: gated_unit's limit (0: silu, below: gelu)
 };
 
 constexpr int kPlain = 0, kScaled = 1, kTail = 2;
@@ -382,7 +382,12 @@ __global__ __launch_bounds__(64 * GM * GN, 1) void gemm_tiled_kernel(TiledArgs g
   TO* c = (TO*)g.c;
   const bool clamped = PAIR && g.limit > 0.f;
   const float top = clamped ? g.limit : INFINITY, lift = clamped ? 1.f : 0.f;
-  const float slope = clamped ? -1.702f * 1.44269504f : -1.44269504f;
+  // the weight exp2(gc (slope + cubic gc^2)): of the sigmoid, or, for gelu_tanh(g) =
+  // g sigmoid(2 sqrt(2 / pi) (g + 0.044715 g^3)), of that one
+  const bool gelu = PAIR && g.limit < 0.f;
+  const float slope = clamped ? -1.702f * 1.44269504f
+                              : (gelu ? -1.59576912160573f * 1.44269504f : -1.44269504f);
+  const float cubic = gelu ? 0.044715f * slope : 0.f;
   if constexpr (FORM == kScaled) {
     // (the barriers of the K loop lie between the factors' writes and these reads)
 #pragma unroll
@@ -411,9 +416,11 @@ __global__ __launch_bounds__(64 * GM * GN, 1) void gemm_tiled_kernel(TiledArgs g
           const float gv = (float)(TO)gate[e], uv = (float)(TO)up[e];
           // 64 values a lane at the very end of the kernel, the matrix cores idle: the
           // hardware's exp2 and reciprocal (an ulp each) instead of a division's ten steps
-          // (gated_unit's two forms: the clamps change nothing without a limit)
+          // (gated_unit's three forms: the clamps change nothing without a limit; far on the
+          // gate's negative side the power is infinite and the reciprocal zero)
           const float gc = fminf(gv, top), uc = fminf(fmaxf(uv, -top), top) + lift;
-          o[e] = gc * __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(gc * slope)) * uc;
+          const float power = gc * fmaf(cubic, gc * gc, slope);
+          o[e] = gc * __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(power)) * uc;
         }
         store4<TO>(c + (int64_t)m * g.N + n, o, g.N - n);
       }

@@ -15,6 +15,7 @@
 // A request's state is read only where a portion does not start at position 0, and is
 // written once a portion, by the thread that owns the element.
 #include "common.h"
+#include <type_traits>
 
 struct BatchView {
   const int* positions;       // [T]
@@ -36,6 +37,9 @@ struct RecurrenceArgs {
   float* out;            // [T, heads*P]
   BatchView b;
   int ld, q_col, k_col, v_col, ldg, heads, kv_heads, N, P, silu;
+  const float2* turn;    // [max_pos, turn_dims / 2]: cosine and sine of a pair's angle, or null
+  int turn_dims;         // leading channels of q and k that are turned, neighbours in pairs
+  float k_scale;         // a factor on k behind its rotation
   const int* chunks;        // [num_chunks, 3]: first token, one past the last, entry
   const int* entry_chunks;  // [B + 1]: the chunks of entry e are [entry_chunks[e], entry_chunks[e+1])
   float* chunk_state;       // [num_chunks, heads, N, P]: local contribution, then start state
@@ -68,6 +72,11 @@ __device__ __forceinline__ float sum_slices(float v) {
   return v;
 }
 
+// The value the other lane of a pair of neighbours holds.
+__device__ __forceinline__ float swap_pair(float v) {
+  return __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), 0xB1, 0xf, 0xf, true));
+}
+
 template <int NI>
 __device__ __forceinline__ void read_rows(const float* p, float (&r)[NI]) {
   if constexpr (NI % 4 == 0) {
@@ -91,7 +100,10 @@ __device__ __forceinline__ void read_rows(const float* p, float (&r)[NI]) {
 // multiply-adds in one wavefront, so a long portion of few entries takes sixteen lanes a
 // column and one column a thread (half the rows a lane, twice the wavefronts), a step of
 // many entries eight lanes and four columns (its states stream in wider rows).
-template <int NI, int CPT, int SL, bool DELTA, bool PER_ROW, int MODE = kRecWhole>
+// TURN: the operands are turned by their token's position as they are staged: channels 2i
+// and 2i + 1 (they stand in neighbouring lanes) by the angle of row `position` of the table,
+// and k is scaled.
+template <int NI, int CPT, int SL, bool DELTA, bool PER_ROW, int MODE = kRecWhole, bool TURN = false>
 __global__ __launch_bounds__(kRecThreads) void recurrence_kernel(RecurrenceArgs a) {
   constexpr int kRecSlices = SL, kRecGroups = kRecThreads / SL;
   constexpr int EPT = kRecStage * SL * NI / kRecThreads;   // elements of q a thread stages
@@ -142,6 +154,8 @@ __global__ __launch_bounds__(kRecThreads) void recurrence_kernel(RecurrenceArgs 
 
   // a stage's operands: from memory into registers (fetch), from there into a buffer (commit)
   float pq[EPT], pk[EPT], pg[PER_ROW ? EPT : 1], pv[VPT], pbeta = 0.f, pgate = 1.f;
+  float2 pt[TURN ? EPT : 1];
+  const int pos0 = TURN ? a.b.positions[first] - first : 0;
   auto fetch = [&](int t0) {
     const int nt = min(kRecStage, end - t0);
     // (element j of a thread is row i % NP of token i / NP in the padded layout: NP is a
@@ -152,10 +166,13 @@ __global__ __launch_bounds__(kRecThreads) void recurrence_kernel(RecurrenceArgs 
       const int tt = i / NP, n = i % NP;
       pq[j] = pk[j] = 0.f;
       if (PER_ROW) pg[j] = 0.f;
+      if (TURN) pt[j] = make_float2(1.f, 0.f);
       if (tt < nt && n < N) {
         const float* row = a.x + (int64_t)(t0 + tt) * a.ld;
-        pq[j] = row[a.q_col + hk * N + n];
+        if (MODE != kRecLocal) pq[j] = row[a.q_col + hk * N + n];     // (a chunk alone gives no o)
         pk[j] = row[a.k_col + hk * N + n];
+        if (TURN && n < a.turn_dims)
+          pt[j] = a.turn[(int64_t)(pos0 + t0 + tt) * (a.turn_dims / 2) + n / 2];
         if (PER_ROW) pg[j] = a.gates[(int64_t)(t0 + tt) * a.ldg + a.heads + h * N + n];
       }
     }
@@ -177,8 +194,16 @@ __global__ __launch_bounds__(kRecThreads) void recurrence_kernel(RecurrenceArgs 
     for (int j = 0; j < EPT; ++j) {
       const int i = j * kRecThreads + threadIdx.x;       // = token * NP + row, padding included
       const int at = (i / NP) * LP + (i % NP) / NI * SP + i % NI;
-      buf[kQ + at] = a.silu ? silu_f(pq[j]) : pq[j];
-      buf[kK + at] = a.silu ? silu_f(pk[j]) : pk[j];
+      if constexpr (TURN) {
+        // (element n's partner of the pair is the neighbouring lane's; EPT x threads is whole
+        // tokens, so the two always hold the same token)
+        const float s = (i % NP) & 1 ? pt[j].y : -pt[j].y;
+        if (MODE != kRecLocal) buf[kQ + at] = fmaf(swap_pair(pq[j]), s, pq[j] * pt[j].x);
+        buf[kK + at] = a.k_scale * fmaf(swap_pair(pk[j]), s, pk[j] * pt[j].x);
+      } else {
+        if (MODE != kRecLocal) buf[kQ + at] = a.silu ? silu_f(pq[j]) : pq[j];
+        buf[kK + at] = a.silu ? silu_f(pk[j]) : pk[j];
+      }
       if (PER_ROW) buf[kG + at] = pg[j];
     }
 #pragma unroll
@@ -284,18 +309,18 @@ __global__ __launch_bounds__(256) void recurrence_combine_kernel(RecurrenceArgs 
   st[idx] = S;
 }
 
-template <int NI, int CPT>
+template <int NI, int CPT, bool TURN>
 static void launch_recurrence_chunked(const RecurrenceArgs& a, int num_entries, int num_chunks,
                                       hipStream_t stream) {
   constexpr int SL = 8, LP = SL * (NI + 4), BC = kRecThreads / SL * CPT;
   const dim3 grid(a.heads, num_chunks, (a.P + BC - 1) / BC);
   const int buf = (kRecStage * (2 * LP + 1 + BC + 1) + 3) / 4 * 4;
   const size_t lds = (size_t)2 * buf * sizeof(float);
-  hipLaunchKernelGGL((recurrence_kernel<NI, CPT, 8, false, false, kRecLocal>), grid,
+  hipLaunchKernelGGL((recurrence_kernel<NI, CPT, 8, false, false, kRecLocal, TURN>), grid,
                      dim3(kRecThreads), lds, stream, a);
   hipLaunchKernelGGL(recurrence_combine_kernel, dim3(a.heads, num_entries, (a.N * a.P + 255) / 256),
                      dim3(256), 0, stream, a);
-  hipLaunchKernelGGL((recurrence_kernel<NI, CPT, 8, false, false, kRecOutput>), grid,
+  hipLaunchKernelGGL((recurrence_kernel<NI, CPT, 8, false, false, kRecOutput, TURN>), grid,
                      dim3(kRecThreads), lds, stream, a);
 }
 
@@ -309,6 +334,7 @@ static int launch_recurrence_cols(const RecurrenceArgs& a, int num_entries, bool
   const size_t lds = (size_t)2 * buf * sizeof(float);
   const void* fn = delta && per_row ? (const void*)recurrence_kernel<NI, CPT, SL, true, true>
                    : delta          ? (const void*)recurrence_kernel<NI, CPT, SL, true, false>
+                   : a.turn ? (const void*)recurrence_kernel<NI, CPT, SL, false, false, kRecWhole, true>
                                     : (const void*)recurrence_kernel<NI, CPT, SL, false, false>;
   if (lds > 64 * 1024 &&
       hipFuncSetAttribute(fn, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds) != hipSuccess)
@@ -317,6 +343,9 @@ static int launch_recurrence_cols(const RecurrenceArgs& a, int num_entries, bool
     hipLaunchKernelGGL((recurrence_kernel<NI, CPT, SL, true, true>), grid, block, lds, stream, a);
   else if (delta)
     hipLaunchKernelGGL((recurrence_kernel<NI, CPT, SL, true, false>), grid, block, lds, stream, a);
+  else if (a.turn)
+    hipLaunchKernelGGL((recurrence_kernel<NI, CPT, SL, false, false, kRecWhole, true>), grid, block,
+                       lds, stream, a);
   else
     hipLaunchKernelGGL((recurrence_kernel<NI, CPT, SL, false, false>), grid, block, lds, stream, a);
   return 0;
@@ -347,6 +376,10 @@ static int launch_recurrence(const RecurrenceArgs& a, int num_entries, bool delt
 // [num_chunks, 3] cuts every entry into runs of tokens (first, one past the last, entry), in
 // order, `entry_chunks` [B + 1] says which are whose, and chunk_state [num_chunks, heads, N,
 // P], chunk_decay [num_chunks, heads] are scratch.
+// `turn` [turn_rows, turn_dims / 2] (cosine, sine), or null: without the delta rule and without
+// `silu`, the first `turn_dims` channels of every q and k head are turned by the row of the
+// token's position, channels 2i and 2i + 1 in pairs, and k is multiplied by k_scale.  (The host
+// sees to it that no position reaches turn_rows.)
 extern "C" int ts_linear_recurrence(const float* x, int ld, int q_col, int k_col, int v_col,
                                     const float* decay, const float* gates, int ldg, float* state,
                                     float* out, const int* positions, const int* entry_of_token,
@@ -354,7 +387,8 @@ extern "C" int ts_linear_recurrence(const float* x, int ld, int q_col, int k_col
                                     int num_entries, int max_q_len, int heads, int kv_heads,
                                     int N, int P, int silu, int delta, int per_row,
                                     const int* chunks, const int* entry_chunks, int num_chunks,
-                                    float* chunk_state, float* chunk_decay, hipStream_t stream) {
+                                    float* chunk_state, float* chunk_decay, const float* turn,
+                                    int turn_dims, float k_scale, hipStream_t stream) {
   if (num_tokens <= 0) return 0;
   if (heads <= 0 || kv_heads <= 0 || heads % kv_heads || N <= 0 || P <= 0)
     TS_FAIL("linear_recurrence: bad sizes heads=%d kv_heads=%d dim=%d vdim=%d", heads, kv_heads, N, P);
@@ -371,17 +405,27 @@ extern "C" int ts_linear_recurrence(const float* x, int ld, int q_col, int k_col
   RecurrenceArgs a{x, decay, gates, state, out,
                    BatchView{positions, entry_of_token, q_start, slot_ids},
                    ld, q_col, k_col, v_col, ldg, heads, kv_heads, N, P, silu,
+                   (const float2*)turn, turn_dims, k_scale,
                    chunks, entry_chunks, chunk_state, chunk_decay};
+  if (turn && (delta || per_row || silu || turn_dims < 2 || turn_dims % 2 || turn_dims > N))
+    TS_FAIL("linear_recurrence: a rotation of %d of %d channels goes with plain operands and without "
+            "the delta rule", turn_dims, N);
+  if (!turn && k_scale != 1.f) TS_FAIL("linear_recurrence: a factor on k comes with a rotation");
   const int ni = (N + 7) / 8;
   if (num_chunks > 0) {
     if (delta) TS_FAIL("linear_recurrence: the delta rule is not linear in S and runs whole");
     if (!chunks || !entry_chunks || !chunk_state || !chunk_decay)
       TS_FAIL("linear_recurrence: chunked without its lists and scratch");
     if (ni > 16) TS_FAIL("linear_recurrence: chunks are built for up to 128 key channels");
-    if (ni <= 2) launch_recurrence_chunked<2, 4>(a, num_entries, num_chunks, stream);
-    else if (ni <= 4) launch_recurrence_chunked<4, 4>(a, num_entries, num_chunks, stream);
-    else if (ni <= 8) launch_recurrence_chunked<8, 4>(a, num_entries, num_chunks, stream);
-    else launch_recurrence_chunked<16, 4>(a, num_entries, num_chunks, stream);
+    auto run = [&](auto turned) {
+      constexpr bool T = decltype(turned)::value;
+      if (ni <= 2) launch_recurrence_chunked<2, 4, T>(a, num_entries, num_chunks, stream);
+      else if (ni <= 4) launch_recurrence_chunked<4, 4, T>(a, num_entries, num_chunks, stream);
+      else if (ni <= 8) launch_recurrence_chunked<8, 4, T>(a, num_entries, num_chunks, stream);
+      else launch_recurrence_chunked<16, 4, T>(a, num_entries, num_chunks, stream);
+    };
+    if (turn) run(std::true_type{});
+    else run(std::false_type{});
     TS_CHECK_LAUNCH("linear_recurrence (chunked)");
     return 0;
   }
@@ -450,7 +494,7 @@ extern "C" int ts_delta_gates(float* qkv, int ld, const float* proj, int ldp, in
 // ---------------------------------------------------------------- norm and gate
 // Each of `groups` equal parts of a row of y is divided by its root mean square, weighed by
 // w (w_len values: one per column of a part, shared by the parts, or one per column of the
-// row) and multiplied by act(gate[gate_col + column]); act: 0 sigmoid, 1 SiLU.
+// row; null: not weighed) and multiplied by act(gate[gate_col + column]); act: 0 sigmoid, 1 SiLU.
 // One wavefront per (row, part).
 template <typename TO>
 __global__ __launch_bounds__(256) void norm_gate_kernel(
@@ -464,14 +508,14 @@ __global__ __launch_bounds__(256) void norm_gate_kernel(
   const int grp = (int)(unit % groups), size = inner / groups;
   const float* yr = y + t * inner + grp * size;
   const float* gr = gate + t * ldgate + gate_col + grp * size;
-  const float* wr = w + (w_len == size ? 0 : grp * size);
+  const float* wr = w ? w + (w_len == size ? 0 : grp * size) : nullptr;
   float ss = 0.f;
   for (int i = lane; i < size; i += kWave) ss = fmaf(yr[i], yr[i], ss);
   const float r = 1.0f / sqrtf(wave_sum(ss) / (float)size + eps);
   TO* o = out + t * inner + grp * size;
   for (int i = lane; i < size; i += kWave) {
     const float g = gr[i];
-    o[i] = from_f32<TO>(yr[i] * r * wr[i] * (act == 0 ? sigmoid_f(g) : silu_f(g)));
+    o[i] = from_f32<TO>(yr[i] * r * (wr ? wr[i] : 1.f) * (act == 0 ? sigmoid_f(g) : silu_f(g)));
   }
 }
 
@@ -480,7 +524,7 @@ extern "C" int ts_norm_gate(const float* y, const float* gate, int ldgate, int g
                             int inner, int groups, int act, float eps, hipStream_t stream) {
   if (rows <= 0) return 0;
   if (inner <= 0 || groups <= 0 || inner % groups || gate_col < 0 || gate_col + inner > ldgate ||
-      (w_len != inner && w_len != inner / groups) || (act != 0 && act != 1))
+      (w && w_len != inner && w_len != inner / groups) || (act != 0 && act != 1))
     TS_FAIL("norm_gate: bad sizes inner=%d groups=%d weight=%d gate columns %d..%d of %d", inner,
             groups, w_len, gate_col, gate_col + inner, ldgate);
   const int64_t units = (int64_t)rows * groups;

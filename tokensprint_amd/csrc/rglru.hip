@@ -24,9 +24,6 @@ struct LruBatch {
 };
 
 __device__ __forceinline__ float sigmoid_f(float v) { return 1.0f / (1.0f + expf(-v)); }
-__device__ __forceinline__ float gelu_tanh_f(float z) {
-  return 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
-}
 
 // ---------------------------------------------------------------- gates
 // A workgroup per (TT tokens, block).  The tokens' inputs of the block lie in LDS; a thread
@@ -217,7 +214,7 @@ __global__ __launch_bounds__(256) void rglru_walk_kernel(
 #pragma unroll 4
   for (int t = first; t < end; ++t) {
     S = fmaf(a[(int64_t)t * width + c], S, x[(int64_t)t * width + c]);
-    out[(int64_t)t * width + c] = from_f32<T>(S * gelu_tanh_f(yproj[(int64_t)t * ld + ycol + c] + yb));
+    out[(int64_t)t * width + c] = from_f32<T>(S * gelu_tanh(yproj[(int64_t)t * ld + ycol + c] + yb));
   }
   *st = S;
 }
@@ -279,7 +276,7 @@ __global__ __launch_bounds__(256) void rglru_output_kernel(
 #pragma unroll 8
   for (int t = first; t < end; ++t) {
     S = fmaf(a[(int64_t)t * width + c], S, x[(int64_t)t * width + c]);
-    out[(int64_t)t * width + c] = from_f32<T>(S * gelu_tanh_f(yproj[(int64_t)t * ld + ycol + c] + yb));
+    out[(int64_t)t * width + c] = from_f32<T>(S * gelu_tanh(yproj[(int64_t)t * ld + ycol + c] + yb));
   }
 }
 

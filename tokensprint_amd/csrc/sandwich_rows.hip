@@ -186,13 +186,150 @@ extern "C" int ts_postnorm_add(float* resid, const void* delta, int delta_type,
   return 0;
 }
 
+// ---------------------------------------------------------------- two outputs, one sum
+// d = a / rms(a) * wa + b / rms(b) * wb, the outputs of two sub-layers that run side by
+// side, each normed by itself; then, where there is a stream, resid += d / rms(d) * post_w and
+// THEN as above; without one d itself goes to `out`.  A row's values of a, b and resid wait in
+// registers between the sums (up to kRowItems a thread; what lies beyond is read again).
+__device__ __forceinline__ float2 block_sum2(float a, float b, float* scratch) {
+  a = wave_sum(a);
+  b = wave_sum(b);
+  const int wave = threadIdx.x / kWave, lane = threadIdx.x % kWave;
+  const int nwaves = (blockDim.x + kWave - 1) / kWave;
+  __syncthreads();
+  if (lane == 0) scratch[2 * wave] = a, scratch[2 * wave + 1] = b;
+  __syncthreads();
+  float2 total = make_float2(0.f, 0.f);
+  for (int w = 0; w < nwaves; ++w) total.x += scratch[2 * w], total.y += scratch[2 * w + 1];
+  return total;
+}
+
+template <typename TA, typename TB, typename TO, int THEN, bool STREAM>
+__global__ __launch_bounds__(1024) void pair_add_kernel(
+    float* __restrict__ resid, const TA* __restrict__ a, const float* __restrict__ wa,
+    const TB* __restrict__ b, const float* __restrict__ wb, float pair_eps,
+    const float* __restrict__ post_w, float post_eps, const float* __restrict__ norm_w,
+    float norm_eps, TO* __restrict__ out, int width) {
+  __shared__ float scratch[32];
+  const int64_t row = blockIdx.x;
+  const int nt = blockDim.x;
+  const TA* ar = a + row * width;
+  const TB* br = b + row * width;
+  float* x = STREAM ? resid + row * width : nullptr;
+  TO* o = out ? out + row * width : nullptr;
+  float dc[kRowItems], bc[kRowItems], xc[kRowItems], wac[kRowItems], wbc[kRowItems];
+  float pc[STREAM ? kRowItems : 1], nc[THEN == kThenNorm ? kRowItems : 1];
+  float sa = 0.f, sb = 0.f;
+#pragma unroll
+  for (int k = 0; k < kRowItems; ++k) {
+    const int i = threadIdx.x + k * nt;
+    const bool in = i < width;
+    dc[k] = in ? to_f32(ar[i]) : 0.f;
+    bc[k] = in ? to_f32(br[i]) : 0.f;
+    wac[k] = in ? wa[i] : 0.f;
+    wbc[k] = in ? wb[i] : 0.f;
+    if (STREAM) {
+      xc[k] = in ? x[i] : 0.f;
+      pc[k] = in ? post_w[i] : 0.f;
+    }
+    if (THEN == kThenNorm) nc[k] = in ? norm_w[i] : 0.f;
+  }
+#pragma unroll
+  for (int k = 0; k < kRowItems; ++k) sa = fmaf(dc[k], dc[k], sa), sb = fmaf(bc[k], bc[k], sb);
+  for (int i = threadIdx.x + kRowItems * nt; i < width; i += nt) {
+    const float va = to_f32(ar[i]), vb = to_f32(br[i]);
+    sa = fmaf(va, va, sa), sb = fmaf(vb, vb, sb);
+  }
+  const float2 ss = block_sum2(sa, sb, scratch);
+  const float ra = inv_rms(ss.x, width, pair_eps), rb = inv_rms(ss.y, width, pair_eps);
+  auto beyond = [&](int i) { return to_f32(ar[i]) * ra * wa[i] + to_f32(br[i]) * rb * wb[i]; };
+  float sd = 0.f;
+#pragma unroll
+  for (int k = 0; k < kRowItems; ++k) {
+    dc[k] = dc[k] * ra * wac[k] + bc[k] * rb * wbc[k];
+    sd = fmaf(dc[k], dc[k], sd);
+  }
+  for (int i = threadIdx.x + kRowItems * nt; i < width; i += nt) {
+    const float v = beyond(i);
+    sd = fmaf(v, v, sd);
+  }
+  if constexpr (!STREAM) {
+#pragma unroll
+    for (int k = 0; k < kRowItems; ++k) {
+      const int i = threadIdx.x + k * nt;
+      if (i < width) o[i] = from_f32<TO>(dc[k]);
+    }
+    for (int i = threadIdx.x + kRowItems * nt; i < width; i += nt) o[i] = from_f32<TO>(beyond(i));
+  } else {
+    const float r = inv_rms(block_sum(sd, scratch), width, post_eps);
+    float sx = 0.f;
+#pragma unroll
+    for (int k = 0; k < kRowItems; ++k) {
+      const int i = threadIdx.x + k * nt;
+      if (i < width) {
+        xc[k] += dc[k] * r * pc[k];
+        x[i] = xc[k];
+        if (THEN == kThenRows) o[i] = from_f32<TO>(xc[k]);
+        sx = fmaf(xc[k], xc[k], sx);
+      }
+    }
+    for (int i = threadIdx.x + kRowItems * nt; i < width; i += nt) {
+      const float v = x[i] + beyond(i) * r * post_w[i];
+      x[i] = v;
+      if (THEN == kThenRows) o[i] = from_f32<TO>(v);
+      sx = fmaf(v, v, sx);
+    }
+    if constexpr (THEN == kThenNorm) {
+      const float r2 = inv_rms(block_sum(sx, scratch), width, norm_eps);
+#pragma unroll
+      for (int k = 0; k < kRowItems; ++k) {
+        const int i = threadIdx.x + k * nt;
+        if (i < width) o[i] = from_f32<TO>(xc[k] * r2 * nc[k]);
+      }
+      // each thread reads back the elements it wrote itself
+      for (int i = threadIdx.x + kRowItems * nt; i < width; i += nt)
+        o[i] = from_f32<TO>(x[i] * r2 * norm_w[i]);
+    }
+  }
+}
+
+// `resid` null: the pair's sum goes to `out`.  Else with `norm_w` the norm of the new stream
+// goes to `out`, with `out` alone the new stream's rows, and without it nothing more.
+extern "C" int ts_pair_add(float* resid, const void* a, int a_type, const float* wa, const void* b,
+                           int b_type, const float* wb, float pair_eps,
+                           const float* post_w, float post_eps, const float* norm_w,
+                           float norm_eps, void* out, int out_type, int rows, int width,
+                           hipStream_t stream) {
+  if (rows <= 0) return 0;
+  if (width <= 0) TS_FAIL("pair_add: bad width %d", width);
+  if (!a || !b || !wa || !wb) TS_FAIL("pair_add: two outputs with a norm weight each");
+  if (resid ? !post_w : (!out || post_w || norm_w))
+    TS_FAIL("pair_add: a stream comes with a norm weight, and without one the sum needs an output");
+  if (norm_w && !out) TS_FAIL("pair_add: a norm without an output");
+  const dim3 grid(rows), block(row_threads(width));
+#define TS_PAIR_LAUNCH(TO, THEN, STREAM)                                                         \
+  hipLaunchKernelGGL((pair_add_kernel<TA, TB, TO, THEN, STREAM>), grid, block, 0, stream, resid, \
+                     (const TA*)a, wa, (const TB*)b, wb, pair_eps, post_w, post_eps,             \
+                     norm_w, norm_eps, (TO*)out, width)
+  TS_DISPATCH_TYPE(a_type, TA, TS_DISPATCH_TYPE(b_type, TB, {
+    if (!resid) {
+      TS_DISPATCH_TYPE(out_type, TO, TS_PAIR_LAUNCH(TO, kThenNothing, false));
+    } else if (!out) {
+      TS_PAIR_LAUNCH(float, kThenNothing, true);
+    } else if (norm_w) {
+      TS_DISPATCH_TYPE(out_type, TO, TS_PAIR_LAUNCH(TO, kThenNorm, true));
+    } else {
+      TS_DISPATCH_TYPE(out_type, TO, TS_PAIR_LAUNCH(TO, kThenRows, true));
+    }
+  }));
+#undef TS_PAIR_LAUNCH
+  TS_CHECK_LAUNCH("pair_add");
+  return 0;
+}
+
 // ---------------------------------------------------------------- a token's own input
 // out[t, j] = gelu_tanh(z[t, j]) * table[ids[t], col + j], j < dim: the gate of what a
 // token's row of a table brings into a layer.  z float32 [T, dim], table [V, ld].
-__device__ __forceinline__ float gelu_tanh(float z) {
-  return 0.5f * z * (1.0f + tanhf(0.79788456080286536f * (z + 0.044715f * z * z * z)));
-}
-
 template <typename TW, typename TO>
 __global__ __launch_bounds__(256) void token_gate_kernel(
     const float* __restrict__ z, const TW* __restrict__ table, const int* __restrict__ ids,

@@ -16,7 +16,7 @@ import torch
 
 from tokensprint_amd.kernels.build import build, find_library
 from tokensprint_amd.kernels.dispatch import default_dispatch
-from tokensprint_amd.kernels.stream import PreparedRows, UnmergedRows
+from tokensprint_amd.kernels.stream import NormedPair, PreparedRows, UnmergedRows
 
 ABI_VERSION = 1
 _TYPE_CODE = {torch.float32: 0, torch.bfloat16: 1}
@@ -194,9 +194,11 @@ class HipOps:
     # and a layer has one dependent kernel less.  The other calls that take activation rows
     # merge first (`_rows`); nothing else can read the rows by mistake, the handle being no
     # tensor.
-    @staticmethod
-    def _rows(x):
-        return x.merged() if x.__class__ is UnmergedRows else x
+    def _rows(self, x):
+        if x.__class__ is UnmergedRows:
+            return x.merged()
+        # two mixers' outputs whose sum nothing has taken into a kernel of its own
+        return self.normed_pair(x, torch.float32) if x.__class__ is NormedPair else x
 
     # ------------------------------------------------------------ rows
     def embed(self, table, token_ids, scale=1.0):
@@ -286,23 +288,27 @@ class HipOps:
                    resid.shape[1], c_float(eps), self._stream())
         return out
 
-    def silu_mul(self, gate_up, limit=None):
+    def silu_mul(self, gate_up, limit=None, act="silu"):
         """gate_up [rows, gate | up] -> silu(gate) * up; with a `limit`, g sigmoid(1.702 g)
-        (u + 1) of g = min(gate, limit) and u = up held between -limit and limit."""
+        (u + 1) of g = min(gate, limit) and u = up held between -limit and limit; with `act`
+        "gelu_tanh", gelu_tanh(gate) * up."""
         self._check("gate_up", gate_up, self._FLOATS, ndim=2)
         rows, two_inner = gate_up.shape
         if two_inner % 2:
             raise ValueError("gate_up needs an even row width (gate half, up half)")
         out = torch.empty(rows, two_inner // 2, dtype=gate_up.dtype, device=self.device)
         self._call(self.lib.ts_silu_mul, _ptr(gate_up), _ptr(out), _TYPE_CODE[gate_up.dtype],
-                   rows, two_inner // 2, self._limit(limit), self._stream())
+                   rows, two_inner // 2, self._unit(limit, act), self._stream())
         return out
 
     @staticmethod
-    def _limit(limit):
-        """A gated unit's limit as the kernels take it (0: there is none)."""
+    def _unit(limit, act):
+        """Which gated unit, in the one number the kernels take: 0 silu(gate) up, a positive
+        number the limit of the clamped unit, a negative one gelu_tanh(gate) up."""
+        if act not in ("silu", "gelu_tanh") or (act != "silu" and limit is not None):
+            raise ValueError(f"gated unit: act={act!r}, limit={limit!r}")
         if limit is None:
-            return c_float(0.0)
+            return c_float(0.0 if act == "silu" else -1.0)
         if not limit > 0:
             raise ValueError(f"a gated unit's limit must be positive, got {limit}")
         return c_float(limit)
@@ -352,10 +358,10 @@ class HipOps:
         self.lib.ts_gemm_library_candidates(8 if on else 1)
         return before
 
-    def gemm_tiled(self, x, weight, out_dtype, pair=False, tile=0, limit=None):
+    def gemm_tiled(self, x, weight, out_dtype, pair=False, tile=0, limit=None, act="silu"):
         """The LDS-tiled product for many rows: x [M, K] bfloat16, weight [N, K] bfloat16
         (with `pair` [2 N, K], gate rows then up rows, and the result is silu(gate) * up, or
-        with a `limit` silu_mul's other form).
+        silu_mul's other forms by `limit` and `act`).
         `tile` 0 lets the sizes choose the tile; another names one (the result is the same
         to the bit)."""
         self._check("x", x, torch.bfloat16, ndim=2)
@@ -366,7 +372,7 @@ class HipOps:
             raise ValueError(f"gemm_tiled: x {tuple(x.shape)}, weight {tuple(weight.shape)}")
         out = torch.empty(M, N, dtype=out_dtype, device=self.device)
         self._call(self.lib.ts_gemm_tiled_bf16, _ptr(x), _ptr(weight), _ptr(out),
-                   _TYPE_CODE[out_dtype], M, N, K, int(pair), tile, self._limit(limit),
+                   _TYPE_CODE[out_dtype], M, N, K, int(pair), tile, self._unit(limit, act),
                    self._stream())
         return out
 
@@ -596,9 +602,9 @@ class HipOps:
                    int(silu_mul), self._stream())
         return out, resid_out
 
-    def linear_silu_mul(self, x, weight, out_dtype, limit=None):
-        """silu(x Wg^T) * (x Wu^T) for weight = [Wg; Wu] stacked by rows -> [M, N/2]; with a
-        `limit` the gated unit is silu_mul's other form."""
+    def linear_silu_mul(self, x, weight, out_dtype, limit=None, act="silu"):
+        """silu(x Wg^T) * (x Wu^T) for weight = [Wg; Wu] stacked by rows -> [M, N/2]; `limit`
+        and `act` choose the gated unit as in silu_mul."""
         x = self._rows(x)
         self._check("x", x, self._FLOATS, ndim=2)
         self._check("weight", weight, self._FLOATS, ndim=2)
@@ -607,14 +613,14 @@ class HipOps:
             raise ValueError(f"linear_silu_mul: x {tuple(x.shape)}, weight {tuple(weight.shape)}")
         inner = weight.shape[0] // 2
         if self._tiled_pair_ok(x, weight, out_dtype):
-            return self.gemm_tiled(x, weight, out_dtype, pair=True, limit=limit)
+            return self.gemm_tiled(x, weight, out_dtype, pair=True, limit=limit, act=act)
         if (self._mfma_ok(x, weight) and out_dtype == torch.bfloat16
                 and not self._library_ok(x, weight, out_dtype)):
             out = torch.empty(M, inner, dtype=out_dtype, device=self.device)
             self._call(self.lib.ts_gemm_mfma_bf16, _ptr(x), _ptr(weight), _ptr(out),
-                       _TYPE_CODE[out_dtype], M, inner, K, 1, self._limit(limit), self._stream())
+                       _TYPE_CODE[out_dtype], M, inner, K, 1, self._unit(limit, act), self._stream())
             return out
-        return self.silu_mul(self.linear(x, weight, out_dtype), limit)
+        return self.silu_mul(self.linear(x, weight, out_dtype), limit, act)
 
     # ------------------------------------------------------------ q/k preparation
     def _qk_args(self, qkv, batch, *, num_heads, kv_in_row, head_dim, q_weight, k_weight, eps,
@@ -1125,6 +1131,41 @@ class HipOps:
                    self._stream())
         return out
 
+    def normed_pair(self, pair, out_dtype):
+        """The sum a `NormedPair` stands for, as a tensor."""
+        return self._pair_add(pair, None, None, 0.0, None, 0.0, out_dtype)
+
+    def pair_postnorm_add(self, resid, pair, post_w, post_eps, norm_w, norm_eps, out_dtype):
+        """resid += d / rms(d) * post_w, in place, of the sum d a `NormedPair` stands for; with
+        `norm_w` the norm of the new resid comes back in `out_dtype`, with `out_dtype` alone
+        its rows (the stream itself if they are float32), else None."""
+        if norm_w is None and out_dtype == torch.float32:
+            self._pair_add(pair, resid, post_w, post_eps, None, 0.0, None)
+            return resid
+        return self._pair_add(pair, resid, post_w, post_eps, norm_w, norm_eps, out_dtype)
+
+    def _pair_add(self, pair, resid, post_w, post_eps, norm_w, norm_eps, out_dtype):
+        a, b = self._rows(pair.a), self._rows(pair.b)
+        self._check("first output", a, self._FLOATS, ndim=2)
+        self._check("second output", b, self._FLOATS, shape=a.shape)
+        rows, W = a.shape
+        self._check("first norm weight", pair.weight_a, torch.float32, shape=(W,))
+        self._check("second norm weight", pair.weight_b, torch.float32, shape=(W,))
+        if resid is not None:
+            self._check("resid", resid, torch.float32, shape=a.shape)
+            self._check("post-norm weight", post_w, torch.float32, shape=(W,))
+        if norm_w is not None:
+            self._check("norm weight", norm_w, torch.float32, shape=(W,))
+        out = None
+        if out_dtype is not None:
+            out = torch.empty(rows, W, dtype=out_dtype, device=self.device)
+        self._call(self.lib.ts_pair_add, _ptr(resid), _ptr(a), _TYPE_CODE[a.dtype],
+                   _ptr(pair.weight_a), _ptr(b), _TYPE_CODE[b.dtype], _ptr(pair.weight_b),
+                   c_float(pair.eps), _ptr(post_w), c_float(post_eps),
+                   _ptr(norm_w), c_float(norm_eps), _ptr(out),
+                   _TYPE_CODE[out_dtype] if out is not None else 0, rows, W, self._stream())
+        return out
+
     def norm_token_shift(self, resid, norm_w, eps, shift_w, batch, state, out_dtype):
         """h = norm(resid); out_t = h_t + (h_(t-1) - h_t) * shift_w.  `state` [slots, width]
         float32 carries a request's last h from step to step."""
@@ -1302,16 +1343,26 @@ class HipOps:
 
     def linear_recurrence(self, x, q_col, k_col, v_col, batch, state, *, heads, kv_heads, dim,
                           vdim, silu_inputs, decay=None, gates=None, per_channel=False,
-                          delta=False):
+                          delta=False, turn=None, k_scale=1.0):
         """Per head and entry, a token at a time: S <- g S; u = v, or (`delta`)
         u = beta (v - S^T k); S <- S + k u^T; o = S^T q -> float32 [T, heads * vdim].
         `x` (float32 [T, ld]) holds q and k (kv_heads x dim; head h reads q/k head
         h // (heads / kv_heads)) and v (heads x vdim) from the given columns, their SiLU taken
         on the way if `silu_inputs`.  g is `decay` [heads] (fixed), or comes with beta from
         `gates` ([T, heads + n] as `delta_gates` lays it out, `per_channel`: one g per row of
-        S).  `state` [slots, heads, dim, vdim] float32 carries S from step to step."""
+        S).  `state` [slots, heads, dim, vdim] float32 carries S from step to step.  `turn`
+        (float32 [positions, pairs, 2], cosines and sines): channels 2i and 2i + 1 of every q
+        and k head, i < pairs, are turned as a pair by the row of their token's position, and
+        k is multiplied by `k_scale` (plain operands, no delta rule)."""
         self._check("x", x, torch.float32, ndim=2)
         T, ld = x.shape
+        if turn is not None:
+            self._check("rotation table", turn, torch.float32, ndim=3)
+            if turn.shape[2] != 2 or 2 * turn.shape[1] > dim:
+                raise ValueError(f"rotation table {tuple(turn.shape)} for {dim} channels")
+            if batch.max_ctx_len > turn.shape[0]:
+                raise ValueError(f"position {batch.max_ctx_len - 1} is beyond the rotation "
+                                 f"table's {turn.shape[0]} rows")
         self._check_state("recurrent state", state, (heads, dim, vdim))
         if decay is not None:
             self._check("decay", decay, torch.float32, shape=(heads,))
@@ -1335,32 +1386,35 @@ class HipOps:
                    batch.num_entries, int(batch.max_q_len), heads, kv_heads, dim, vdim,
                    int(bool(silu_inputs)), int(bool(delta)), int(bool(per_channel)),
                    _ptr(chunks), _ptr(entry_chunks), num_chunks, _ptr(scratch), _ptr(decays),
+                   _ptr(turn), 2 * turn.shape[1] if turn is not None else 0, c_float(k_scale),
                    self._stream())
         return out
 
     def norm_gate(self, y, gate_rows, gate_col, norm_w, *, groups, gate, eps, out_dtype):
         """Each of `groups` equal parts of a row of y (float32) over its root mean square,
         times norm_w (one value per column of a part, shared by the parts, or one per column
-        of the row), times sigmoid or SiLU (`gate`) of columns [gate_col, gate_col + width) of
+        of the row; None: not weighed), times sigmoid or SiLU (`gate`) of columns [gate_col, gate_col + width) of
         `gate_rows` (float32)."""
         self._check("y", y, torch.float32, ndim=2)
         T, inner = y.shape
         self._check("gate rows", gate_rows, torch.float32, ndim=2)
-        self._check("norm weight", norm_w, torch.float32, ndim=1)
+        if norm_w is not None:
+            self._check("norm weight", norm_w, torch.float32, ndim=1)
         if gate not in ("sigmoid", "silu"):
             raise ValueError(f"norm_gate: gate {gate!r}; built are sigmoid and silu")
         if gate_rows.shape[0] != T:
             raise ValueError("norm_gate: row counts differ")
         out = torch.empty(T, inner, dtype=out_dtype, device=self.device)
         self._call(self.lib.ts_norm_gate, _ptr(y), _ptr(gate_rows), gate_rows.shape[1],
-                   int(gate_col), _ptr(norm_w), norm_w.shape[0], _ptr(out), _TYPE_CODE[out_dtype],
+                   int(gate_col), _ptr(norm_w), norm_w.shape[0] if norm_w is not None else 0,
+                   _ptr(out), _TYPE_CODE[out_dtype],
                    T, inner, int(groups), 0 if gate == "sigmoid" else 1, c_float(eps),
                    self._stream())
         return out
 
     # ------------------------------------------------------------ routed experts
     def route_experts(self, logits, *, top, group_count=1, group_keep=1, scores="softmax",
-                      normalize=True, correction=None, weight_scale=1.0):
+                      normalize=True, correction=None, weight_scale=1.0, bias=None):
         """Router logits (float32 [T, experts]) -> float32 [T, experts]: a token's weight for
         each of its `top` experts (softmax score over the chosen scores' sum), zero elsewhere.
         Only experts of the `group_keep` best of `group_count` groups of neighbours can be
@@ -1368,17 +1422,20 @@ class HipOps:
         the sigmoid of its logit; `normalize` False: the weights are the chosen scores as
         they are.  `correction` (float32 [experts]): groups and experts are ranked by score +
         correction (softmax scores), the weights stay the scores; `weight_scale`: a factor on
-        the weights."""
+        the weights.  `bias` (float32 [experts]) is added to the logits first."""
         if scores not in ("softmax", "sigmoid"):
             raise ValueError(f"route_experts: scores={scores!r}")
         self._check("router logits", logits, torch.float32, ndim=2)
         T, E = logits.shape
         if correction is not None:
             self._check("correction", correction, torch.float32, shape=(E,))
+        if bias is not None:
+            self._check("router bias", bias, torch.float32, shape=(E,))
         weights = torch.empty(T, E, dtype=torch.float32, device=self.device)
         self._call(self.lib.ts_route_experts, _ptr(logits), _ptr(weights), T, E, int(top),
                    int(group_count), int(group_keep), int(scores == "sigmoid"),
-                   int(bool(normalize)), _ptr(correction), c_float(weight_scale), self._stream())
+                   int(bool(normalize)), _ptr(correction), c_float(weight_scale), _ptr(bias),
+                   self._stream())
         return weights
 
     def expert_activation(self, gate_up, weights, inner, limit, out_dtype, weighted_input=False,

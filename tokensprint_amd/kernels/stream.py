@@ -80,6 +80,20 @@ class StreamRows:
     rows: torch.Tensor
 
 
+@dataclass(frozen=True)
+class NormedPair:
+    """What two mixers side by side may return in place of a tensor: norm_a(a) + norm_b(b),
+    each output over its root mean square (eps inside the root) times its weight.
+    A block that norms the sum and adds it to the stream lets one kernel do all of it
+    (`pair_postnorm_add`); `normed_pair` of the provider gives the tensor to anyone else."""
+
+    a: torch.Tensor
+    weight_a: torch.Tensor
+    b: torch.Tensor
+    weight_b: torch.Tensor
+    eps: float
+
+
 class UnmergedRows:
     """What `attend(defer_merge=True)` may return in place of a tensor: a decode step's
     attention output whose key splits have not been merged yet.  It is deliberately no

@@ -8,7 +8,7 @@ from __future__ import annotations
 
 import torch
 
-from tokensprint_amd.kernels.stream import (NormAhead, NormedRows, RowsAhead, StreamRows,
+from tokensprint_amd.kernels.stream import (NormAhead, NormedPair, NormedRows, RowsAhead, StreamRows,
                                             fused_rmsnorm_of)
 from tokensprint_amd.parts.base import (BLOCKS, FEED_FORWARDS, FILTERS, MIXERS, NORMS, SIDES, Block,
                                         StreamFilter, TensorDecl, SlotStateNeed, register)
@@ -47,60 +47,90 @@ class PreNormBlock(Block):
 @register(BLOCKS, "sandwich_norm")
 class SandwichNormBlock(Block):
     """A norm before and one after each sub-layer:
-    x = x + post1(mixer(filter(norm1(x)))); x = x + post2(ffn(norm2(x))).
-    The filter (what the mixer reads passes through it, e.g. a token shift) and the
-    feed-forward with its two norms may be left out.  With RMS norms the add of the mixer's
-    normalised output and the norm in front of the feed-forward are one kernel, and so are
-    the norm in front of the mixer and the filter; the stream leaves the block summed up
-    (no delta is handed on)."""
+    x = x + post1(mixer(filter(norm1(x)))); x = x + post2(ffn(norm2(x))); then, where the layer
+    has a side input, x = x + post3(side(x, tokens)).
+    The filter (what the mixer reads passes through it, e.g. a token shift), the feed-forward
+    with its two norms and the side input with its norm may be left out.  With RMS norms the
+    add of a sub-layer's normalised output and whatever reads the stream next are one kernel:
+    the norm in front of the feed-forward, the rows of the side input's product, or the norm
+    in front of the next layer's mixer (where that layer is of a kind that asks for it); and
+    so are the norm in front of the mixer and the filter.  The stream leaves the block summed
+    up (no delta is handed on)."""
 
     ROLES = {"mixer_norm": (NORMS, True), "mixer_filter": (FILTERS, False),
              "mixer": (MIXERS, True), "mixer_post_norm": (NORMS, True),
              "ffn_norm": (NORMS, False), "feed_forward": (FEED_FORWARDS, False),
-             "ffn_post_norm": (NORMS, False)}
+             "ffn_post_norm": (NORMS, False), "side": (SIDES, False),
+             "side_post_norm": (NORMS, False)}
 
     def __init__(self, parts, ctx):
         super().__init__(parts, ctx)
         ffn = (self.ffn_norm, self.feed_forward, self.ffn_post_norm)
         if any(p is None for p in ffn) and any(p is not None for p in ffn):
             raise ValueError("sandwich_norm: a feed-forward comes with both of its norms")
+        if (self.side is None) != (self.side_post_norm is None):
+            raise ValueError("sandwich_norm: a side input and its norm come together")
 
-    def _post_add(self, resid, out, post, then=None):
-        """resid += post(out); then, if given, the norm `then` of the sum."""
-        ops = self.ctx.ops
+    def entry_hint(self):
+        fused = fused_rmsnorm_of(self.mixer_norm) if self.mixer_filter is None else None
+        return None if fused is None else NormAhead(fused[0], fused[1])
+
+    def _post_add(self, resid, out, post, then=None, rows=False):
+        """resid += post(out); then, if given, the norm `then` (weight, eps) of the sum, or with
+        `rows` the sum's rows in the activation dtype."""
+        ops, dtype = self.ctx.ops, self.ctx.dtype
         fused = fused_rmsnorm_of(post)
-        nxt = fused_rmsnorm_of(then) if then is not None else None
-        if fused is not None and (then is None or nxt is not None):
-            if then is None:
-                ops.postnorm_add(resid, out, fused[0], fused[1])
-                return None
-            return ops.postnorm_add_norm(resid, out, fused[0], fused[1], nxt[0], nxt[1],
-                                         self.ctx.dtype)
-        # another kind of norm: its own forward, the add through the next norm (or, with
-        # none to follow, through the same norm once more, whose output is dropped)
-        normed = post.forward(out)
-        if then is not None:
-            return then.add_forward(resid, normed)
-        post.add_forward(resid, normed)
+        weight, eps = then or (None, 0.0)
+        if isinstance(out, NormedPair):
+            if fused is not None:
+                return ops.pair_postnorm_add(resid, out, fused[0], fused[1], weight, eps,
+                                             dtype if then or rows else None)
+            out = ops.normed_pair(out, torch.float32)
+        if fused is None:            # another kind of norm: its own forward, then a plain add
+            ops.stream_add(resid, post.forward(out), None, None)
+            if then:
+                return ops.rmsnorm(resid, weight, eps, dtype)
+            return ops.stream_rows(resid, dtype) if rows else None
+        if then:
+            return ops.postnorm_add_norm(resid, out, fused[0], fused[1], weight, eps, dtype)
+        if rows:
+            return ops.postnorm_add_rows(resid, out, fused[0], fused[1], dtype)
+        ops.postnorm_add(resid, out, fused[0], fused[1])
         return None
 
     def forward(self, resid, delta, batch, cache, write_cache, next_hint=None):
-        if delta is not None:
-            # a block in front that hands on a delta (this one gives no entry hint, so it is
-            # a plain tensor): added through the mixer's norm, whose output is not used
-            self.mixer_norm.add_forward(resid, delta)
-        if self.mixer_filter is not None:
+        if isinstance(delta, NormedRows):
+            h = delta.rows
+        elif self.mixer_filter is not None:
+            if delta is not None:
+                # a block in front that hands on a delta (with a filter this one gives no entry
+                # hint, so it is a plain tensor): added through the mixer's norm, whose output
+                # is not used
+                self.mixer_norm.add_forward(resid, delta)
             h = self.mixer_filter.forward_from_stream(resid, self.mixer_norm, batch, cache)
         else:
-            h = self.mixer_norm.forward(resid)
+            h = self.mixer_norm.forward(resid) if delta is None \
+                else self.mixer_norm.add_forward(resid, delta)
+        # the norm the next block opens with, for this block's last add (a row that enters in
+        # front of that block would have to be added first)
+        ahead = (next_hint.norm_weight, next_hint.eps) \
+            if isinstance(next_hint, NormAhead) and next_hint.row is None else None
+        side_reads = self.side is not None
         out = self.mixer.forward(h, batch, cache, write_cache)
         if self.feed_forward is None:
-            self._post_add(resid, out, self.mixer_post_norm)
-            return resid, None
-        h = self._post_add(resid, out, self.mixer_post_norm, then=self.ffn_norm)
-        out = self.feed_forward.forward(h, batch)
-        self._post_add(resid, out, self.ffn_post_norm)
-        return resid, None
+            h = self._post_add(resid, out, self.mixer_post_norm,
+                               None if side_reads else ahead, rows=side_reads)
+        else:
+            norm = fused_rmsnorm_of(self.ffn_norm)
+            h = self._post_add(resid, out, self.mixer_post_norm, norm)
+            if norm is None:
+                h = self.ffn_norm.forward(resid)
+            out = self.feed_forward.forward(h, batch)
+            h = self._post_add(resid, out, self.ffn_post_norm,
+                               None if side_reads else ahead, rows=side_reads)
+        if side_reads:
+            h = self._post_add(resid, self.side.forward(h, batch), self.side_post_norm, ahead)
+        return resid, NormedRows(h, False) if ahead else None
 
 
 @register(BLOCKS, "post_norm")

@@ -16,11 +16,12 @@ from tokensprint_amd.parts.base import FEED_FORWARDS, FeedForward, TensorDecl, r
 @register(FEED_FORWARDS, "swiglu")
 class SwiGLU(StreamProducts, FeedForward):
     """down(silu(gate(h)) * up(h)); with a `limit`, down(g sigmoid(1.702 g) (u + 1)) of g =
-    min(gate(h), limit) and u = up(h) held between -limit and limit.
+    min(gate(h), limit) and u = up(h) held between -limit and limit; with `act` "gelu_tanh",
+    down(gelu_tanh(gate(h)) * up(h)).
 
     params: prefix, inner_dim, names (the tensors' names behind the prefix, gate, up and
     down; default 'gate_proj.weight', 'up_proj.weight', 'down_proj.weight'), limit (None: the
-    plain unit), wide_output (the result leaves in float32, for a block that norms it)."""
+    plain unit), act ("silu", the default, or "gelu_tanh"), wide_output (the result leaves in float32, for a block that norms it)."""
 
     def __init__(self, params, ctx):
         super().__init__(params, ctx)
@@ -29,6 +30,13 @@ class SwiGLU(StreamProducts, FeedForward):
         self.names = tuple(self.prefix + n for n in params.get(
             "names", ("gate_proj.weight", "up_proj.weight", "down_proj.weight")))
         self.limit = float(params["limit"]) if params.get("limit") is not None else None
+        self.act = params.get("act", "silu")
+        if self.act not in ("silu", "gelu_tanh") or (self.act != "silu" and self.limit is not None):
+            raise ValueError(f"{self.prefix}: act={self.act!r}, limit={self.limit}")
+        #: what tells the products' gated unit from the plain one
+        self.form = {} if self.limit is None else {"limit": self.limit}
+        if self.act != "silu":
+            self.form["act"] = self.act
         self.out_dtype = torch.float32 if params.get("wide_output") else ctx.dtype
         self.w_gate_up = self.w_down = None
 
@@ -45,21 +53,20 @@ class SwiGLU(StreamProducts, FeedForward):
         self.w_down = get(self.names[2])
 
     def stream_hint(self, norm):
-        if self.limit is not None:
+        if self.form:
             return None          # the products with the norm inside know the plain unit only
         return self.first_product_hint(norm, self.w_gate_up, silu_mul=True)
 
     def forward_from_stream(self, resid, delta, norm, batch, hint=None):
         fused = fused_rmsnorm_of(norm)
-        if fused is None or self.limit is not None:
+        if fused is None or self.form:
             return super().forward_from_stream(resid, delta, norm, batch)
         act, resid = self.ops.norm_linear(resid, delta, fused[0], fused[1], self.w_gate_up,
                                           self.ctx.dtype, silu_mul=True)
         return self.last_product(act, self.w_down, resid, hint), resid
 
     def forward(self, h, batch):
-        form = {} if self.limit is None else {"limit": self.limit}
-        act = self.ops.linear_silu_mul(h, self.w_gate_up, self.ctx.dtype, **form)
+        act = self.ops.linear_silu_mul(h, self.w_gate_up, self.ctx.dtype, **self.form)
         return self.ops.linear(act, self.w_down, self.out_dtype)
 
 
@@ -158,11 +165,12 @@ class RoutedExperts(StreamProducts, FeedForward):
     router's outputs is added to the scores for the choice of groups and experts only: the
     weights are the scores without it); `weight_scale` (a factor on the weights);
     `shared_inner` (one more gated unit, '<prefix>shared.*', that every token uses with the
-    weight one: its rows and columns join the experts' two products).
+    weight one: its rows and columns join the experts' two products); `router_bias` (a vector
+    '<prefix>router.b' is added to the router's logits).
 
     params: prefix, inner_dim (of one expert), experts, top, group_count, group_keep (default
     one group), limit, scores, normalize, gated, identity, correction, weight_scale,
-    shared_inner."""
+    shared_inner, router_bias."""
 
     def __init__(self, params, ctx):
         super().__init__(params, ctx)
@@ -189,11 +197,14 @@ class RoutedExperts(StreamProducts, FeedForward):
         if (self.shared_inner or self.identity) and self.gated != "silu":
             raise ValueError(f"{self.prefix}: a shared expert and identity experts come with "
                              "gated='silu'")
-        self.w_router = self.w_gate_up = self.w_down = self.correction = None
+        self.router_biased = bool(p.get("router_bias", False))
+        self.w_router = self.w_gate_up = self.w_down = self.correction = self.router_bias = None
 
     def tensors(self):
         W, I, pre = self.ctx.width, self.inner, self.prefix
         t = {pre + "router": TensorDecl((self.outputs, W))}
+        if self.router_biased:
+            t[pre + "router.b"] = TensorDecl((self.outputs,), role="vector", init=(-0.5, 0.5))
         for e in range(self.experts):
             t[f"{pre}e{e}.gate"] = TensorDecl((I, W))
             t[f"{pre}e{e}.up"] = TensorDecl((I, W))
@@ -217,6 +228,8 @@ class RoutedExperts(StreamProducts, FeedForward):
         if self.shared_inner:
             rows += [get(pre + "shared.gate"), get(pre + "shared.up")]
             cols.append(get(pre + "shared.down"))
+        if self.router_biased:
+            self.router_bias = get(pre + "router.b").float().contiguous()
         if self.corrected:
             self.correction = get(pre + "correction").float().contiguous()
         if len({r.dtype for r in rows + cols}) != 1:
@@ -238,6 +251,8 @@ class RoutedExperts(StreamProducts, FeedForward):
             more["correction"] = self.correction
         if self.weight_scale != 1.0:
             more["weight_scale"] = self.weight_scale
+        if self.router_biased:
+            more["bias"] = self.router_bias
         weights = ops.route_experts(logits, top=self.top, group_count=self.group_count,
                                     group_keep=self.group_keep, scores=self.scores,
                                     normalize=self.normalize, **more)    # [T, outputs]

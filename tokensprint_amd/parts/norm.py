@@ -11,7 +11,9 @@ class RMSNorm(Norm):
     """params: dim, eps, weight (checkpoint name), one_plus (the checkpoint stores the weight
     around zero and the norm multiplies by 1 + w; the sum is made once, when the weight is
     loaded, in float32), scalar (the checkpoint holds one number for all coordinates; it is
-    spread over `dim` values when it is loaded, so every fused form of the norm serves it)."""
+    spread over `dim` values when it is loaded, so every fused form of the norm serves it),
+    scale (a factor on the norm's output, made part of the weight when it is loaded, in float32;
+    in front of a head it is a factor on the logits)."""
 
     def __init__(self, params, ctx):
         super().__init__(params, ctx)
@@ -20,6 +22,7 @@ class RMSNorm(Norm):
         self.weight_name = params["weight"]
         self.one_plus = bool(params.get("one_plus", False))
         self.scalar = bool(params.get("scalar", False))
+        self.scale = float(params.get("scale", 1.0))
         self.weight = None
 
     def tensors(self):
@@ -32,6 +35,8 @@ class RMSNorm(Norm):
             self.weight = self.weight.float().reshape(1).expand(self.dim).contiguous()
         if self.one_plus:
             self.weight = (self.weight.float() + 1.0).contiguous()
+        if self.scale != 1.0:
+            self.weight = (self.weight.float() * self.scale).contiguous()
 
     def fused_rmsnorm(self):
         return self.weight, self.eps

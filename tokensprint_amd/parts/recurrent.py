@@ -22,18 +22,22 @@ import math
 
 import torch
 
-from tokensprint_amd.kernels.stream import StreamProducts, fused_rmsnorm_of
+from tokensprint_amd.kernels.stream import NormedPair, StreamProducts, fused_rmsnorm_of
 from tokensprint_amd.parts.base import (MIXERS, Mixer, SlotStateNeed, TensorDecl, build_part,
                                         flat_needs, register)
 
 
-@register(MIXERS, "lightning_attention")
-class LightningAttention(Mixer):
-    """q, k, v = silu of their projections, head by head; S <- decay_h S + k v^T, o = S^T q;
-    the heads together pass an RMS norm (weight '<prefix>norm') and a sigmoid gate, then the
-    output projection.
+class FixedDecayAttention(Mixer):
+    """Linear attention with a fixed decay per head: S <- decay_h S + k v^T, o = S^T q, with q,
+    k, v and a gate from one product; o passes an RMS norm and the gate, then the output
+    projection.  What the kinds differ in: SiLU on q, k and v or not, a rotation of q and k (and
+    a factor on k behind it), the norm's parts and weight, the gate's function.
 
     params: prefix, heads, dim, vdim, decay (one per head), eps, state (name of its state)."""
+
+    silu_inputs = False
+    gate = "silu"
+    norm_weighted = False        # '<prefix>norm', a value per column of all heads
 
     def __init__(self, params, ctx):
         super().__init__(params, ctx)
@@ -48,28 +52,39 @@ class LightningAttention(Mixer):
         self.decay = torch.tensor(decay, dtype=torch.float32, device=ctx.device)
         self.qk, self.inner = self.heads * self.dim, self.heads * self.vdim
         self.w_in = self.w_o = self.norm_w = None
+        self.norm_groups = self.heads      # equal parts of a row that are normed by themselves
+        self.turning = {}                  # further keywords of `ops.linear_recurrence`
 
     def tensors(self):
         W, pre = self.ctx.width, self.prefix
-        return {pre + "q": TensorDecl((self.qk, W)), pre + "k": TensorDecl((self.qk, W)),
-                pre + "v": TensorDecl((self.inner, W)), pre + "g": TensorDecl((self.inner, W)),
-                pre + "norm": TensorDecl((self.inner,), role="vector"),
-                pre + "o": TensorDecl((W, self.inner))}
+        t = {pre + "q": TensorDecl((self.qk, W)), pre + "k": TensorDecl((self.qk, W)),
+             pre + "v": TensorDecl((self.inner, W)), pre + "g": TensorDecl((self.inner, W)),
+             pre + "o": TensorDecl((W, self.inner))}
+        if self.norm_weighted:
+            t[pre + "norm"] = TensorDecl((self.inner,), role="vector")
+        return t
+
+    def laid_out(self, w):
+        """The rows of a q or k projection in the order the recurrence wants them."""
+        return w
 
     def load(self, get):
         pre = self.prefix
         rows = [get(pre + n) for n in "qkvg"]
         if len({r.dtype for r in rows}) != 1:
             raise ValueError(f"{pre}: projection weights are stored in different dtypes")
+        rows[0], rows[1] = self.laid_out(rows[0]), self.laid_out(rows[1])
         self.w_in = torch.cat(rows, dim=0).contiguous()
-        self.w_o, self.norm_w = get(pre + "o"), get(pre + "norm")
+        self.w_o = get(pre + "o")
+        if self.norm_weighted:
+            self.norm_w = get(pre + "norm")
 
     def cache_need(self):
         return SlotStateNeed((self.heads, self.dim, self.vdim), torch.float32, self.state_name)
 
     def forward(self, h, batch, cache, write_cache):
         if cache is None or self.state_name not in cache.states:
-            raise RuntimeError(f"{self.prefix}: lightning attention needs its per-request state")
+            raise RuntimeError(f"{self.prefix}: linear attention needs its per-request state")
         if not write_cache:
             raise RuntimeError(f"{self.prefix}: a recurrence cannot read another run's state")
         ops = self.ops
@@ -77,10 +92,44 @@ class LightningAttention(Mixer):
         o = ops.linear_recurrence(
             proj, 0, self.qk, 2 * self.qk, batch, cache.states[self.state_name],
             heads=self.heads, kv_heads=self.heads, dim=self.dim, vdim=self.vdim,
-            silu_inputs=True, decay=self.decay)
-        gated = ops.norm_gate(o, proj, 2 * self.qk + self.inner, self.norm_w, groups=1,
-                              gate="sigmoid", eps=self.eps, out_dtype=self.ctx.dtype)
+            silu_inputs=self.silu_inputs, decay=self.decay, **self.turning)
+        gated = ops.norm_gate(o, proj, 2 * self.qk + self.inner, self.norm_w,
+                              groups=self.norm_groups, gate=self.gate, eps=self.eps,
+                              out_dtype=self.ctx.dtype)
         return ops.linear(gated, self.w_o, torch.float32)
+
+
+@register(MIXERS, "lightning_attention")
+class LightningAttention(FixedDecayAttention):
+    """q, k, v = silu of their projections; the heads together pass an RMS norm (weight
+    '<prefix>norm') and a sigmoid gate."""
+
+    silu_inputs = True
+    gate = "sigmoid"
+    norm_weighted = True
+
+    def __init__(self, params, ctx):
+        super().__init__(params, ctx)
+        self.norm_groups = 1
+
+
+@register(MIXERS, "retention")
+class Retention(FixedDecayAttention):
+    """q and k are rotated by their positions (leading dimensions of every head), k is
+    multiplied by dim^-1/2 behind the rotation; each head's o is divided by its root mean
+    square, without a weight, and multiplied by the SiLU of its gate.
+
+    Further params: position (a 'rope_interleaved' encoding with a table; its `layout` orders the
+    channels of q and k, and so the rows of the state)."""
+
+    def __init__(self, params, ctx):
+        super().__init__(params, ctx)
+        self.position = ctx.positions[params["position"]]
+        self.turning = {"turn": self.position.pair_table(), "k_scale": float(self.dim) ** -0.5}
+
+    def laid_out(self, w):
+        order = torch.tensor(self.position.layout(self.dim), device=w.device)
+        return w.view(self.heads, self.dim, -1)[:, order].reshape(self.qk, -1)
 
 
 @register(MIXERS, "gated_delta")
@@ -298,9 +347,13 @@ class RealGatedLRU(StreamProducts, Mixer):
 @register(MIXERS, "side_by_side")
 class SideBySide(Mixer):
     """Two mixers that read the same input; the result is left_scale * left + right_scale *
-    right.  Each keeps what it needs in the run's cache view (at most one of them pages).
+    right.  Each keeps what it needs in the run's cache view (at most one of them pages).  With
+    `norms` each output is normed over the width first (RMS norm, a weight each), and the
+    result comes back as a `NormedPair`, which a block that norms its mixer's output can take
+    into the kernel of that norm.
 
-    params: left, right (PartSpec of a mixer each), left_scale, right_scale."""
+    params: left, right (PartSpec of a mixer each), left_scale, right_scale, norms (None, or the
+    two weights' tensor names), norm_eps."""
 
     def __init__(self, params, ctx):
         self.left = self.right = None
@@ -309,6 +362,8 @@ class SideBySide(Mixer):
         self.right = build_part(MIXERS, params["right"], ctx)
         self.left_scale, self.right_scale = float(params["left_scale"]), float(params["right_scale"])
         self.capturable = self.left.capturable and self.right.capturable
+        self.norms, self.norm_eps = params.get("norms"), float(params.get("norm_eps", 0.0))
+        self.w_left = self.w_right = None
 
     @property
     def ops(self):
@@ -322,17 +377,23 @@ class SideBySide(Mixer):
                 side.ops = provider
 
     def tensors(self):
-        return {**self.left.tensors(), **self.right.tensors()}
+        own = {name: TensorDecl((self.ctx.width,), role="vector") for name in self.norms or ()}
+        return {**self.left.tensors(), **self.right.tensors(), **own}
 
     def load(self, get):
         self.left.load(get)
         self.right.load(get)
+        if self.norms:
+            # (the scales made part of the weights, in float32)
+            self.w_left = (get(self.norms[0]).float() * self.left_scale).contiguous()
+            self.w_right = (get(self.norms[1]).float() * self.right_scale).contiguous()
 
     def held_tensors(self):
-        return self.left.held_tensors() + self.right.held_tensors()
+        return super().held_tensors() + self.left.held_tensors() + self.right.held_tensors()
 
     def step_read_tensors(self):
-        return self.left.step_read_tensors() + self.right.step_read_tensors()
+        return super().held_tensors() + self.left.step_read_tensors() \
+            + self.right.step_read_tensors()
 
     def cache_need(self):
         return flat_needs((self.left.cache_need(), self.right.cache_need())) or None
@@ -340,4 +401,6 @@ class SideBySide(Mixer):
     def forward(self, h, batch, cache, write_cache):
         a = self.left.forward(h, batch, cache, write_cache)
         b = self.right.forward(h, batch, cache, write_cache)
+        if self.norms:
+            return NormedPair(a, self.w_left, b, self.w_right, self.norm_eps)
         return self.ops.scaled_sum(a, self.left_scale, b, self.right_scale)
