@@ -485,10 +485,46 @@ def fubepel_configs(s):
     return config(ff), zono
 
 
+def sisepel_configs(s):
+    """(Sisepel, Palelix) at the width, depth, vocabulary and number of matrix parameters of
+    the size `s`.  Sisepel: in every layer windowed attention beside retention with as many
+    heads and channels as Palelix's lightning attention has, and a side input of a head's size;
+    routed experts (8, of which a token uses 2, beside a shared one) in every second layer and a
+    dense feed-forward in the others; the dense one's inner size takes up what is left."""
+    import math
+    from tokensprint_amd.weights.random_init import declared_tensors
+    hd, heads, kv = s["head_dim"], s["heads"], s["kv_heads"]
+    pale = palelix_configs(s)[0]
+    expert_ff = pale["layers"][1]["mlp"]["expert"]["ff"] // 2
+    mixer = {"left": {"heads": heads, "kv_heads": kv, "dim": hd, "vdim": hd, "scale": hd ** -0.5,
+                      "softcap": 50.0, "mask": {"size": s["window"]},
+                      "rot": {"base": 5e5, "dims": hd // 2,
+                              "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0,
+                                          "original": 8192}}},
+             "right": {"heads": heads, "dim": hd, "vdim": hd, "rot": {"base": 1e4, "dims": hd},
+                       "decay": [1.0 - 2.0 ** (-(3 + 6 * i / max(heads - 1, 1)))
+                                 for i in range(heads)]}}
+    moe = {"kind": "moe", "expert": {"ff": expert_ff}, "router": {"experts": 8, "top": 2},
+           "shared": {"ff": expert_ff}}
+
+    def config(ff):
+        return {"architecture": "Sisepel", "width": s["width"], "vocab": s["vocab"],
+                "norm": {"eps": 1e-6}, "token_side": {"dim": hd}, "logit_scale": 0.5,
+                "layers": [{"type": "parallel", "mixer": mixer,
+                            "mlp": moe if i % 2 else {"kind": "dense", "ff": ff}}
+                           for i in range(s["layers"])]}
+
+    def count(raw):
+        return sum(math.prod(d.shape) for d in declared_tensors(raw).values())
+    spare = count(pale) - count(config(64))
+    ff = 64 + max(0, round(spare / (3 * s["width"] * -(-s["layers"] // 2)) / 64)) * 64
+    return config(ff), pale
+
+
 #: design -> (its configuration and that of the closest design at equal size, that design)
 COMPARISONS = {"zonopel": (compare_configs, "qwen3"), "palelix": (palelix_configs, "zonopel"),
                "zolorax": (zolorax_configs, "zonopel"), "pinedra": (pinedra_configs, "zolorax"),
-               "fubepel": (fubepel_configs, "zonopel")}
+               "fubepel": (fubepel_configs, "zonopel"), "sisepel": (sisepel_configs, "palelix")}
 
 
 def chosen_design(args, what):
@@ -658,6 +694,11 @@ def main() -> int:
     ap.add_argument("--compare-fubepel", action="store_true",
                     help="instead of the benchmark: prefill and decode throughput of Fubepel "
                          "beside Zonopel at equal sizes, with the time of every kind of kernel")
+    ap.add_argument("--compare-sisepel", action="store_true",
+                    help="instead of the benchmark: prefill and decode throughput of Sisepel "
+                         "beside Palelix at equal sizes, with the time of every kind of kernel")
+    ap.add_argument("--profile-sisepel", default=None, choices=["prefill", "decode"],
+                    help="as --profile-zonopel, for the Sisepel model of --compare-size")
     ap.add_argument("--profile-fubepel", default=None, choices=["prefill", "decode"],
                     help="as --profile-zonopel, for the Fubepel model of --compare-size")
     ap.add_argument("--profile-pinedra", default=None, choices=["prefill", "decode"],

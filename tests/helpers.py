@@ -563,3 +563,130 @@ def write_fubepel_model(folder, cfg, seed, dtype, std=0.2, sharpen=3.0):
             tensors[name] = (tensors[name].float() * sharpen).to(tensors[name].dtype)
     save_file(tensors, str(file))
     return d
+
+
+# ------------------------------------------------------------------ Sisepel
+
+
+def sisepel_scaling(factor, low, high, original):
+    return {"factor": factor, "low": low, "high": high, "original": original}
+
+
+def sisepel_attention(*, heads, kv_heads, dim, vdim, scale, window, softcap, base, rot_dims,
+                      scaling=None):
+    left = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "scale": scale,
+            "rot": {"base": base, "dims": rot_dims}}
+    if scaling is not None:
+        left["rot"]["scaling"] = scaling
+    if window is not None:
+        left["mask"] = {"size": window}
+    if softcap is not None:
+        left["softcap"] = softcap
+    return left
+
+
+def sisepel_retention(*, dim, vdim, decay, base, rot_dims):
+    return {"heads": len(decay), "dim": dim, "vdim": vdim, "decay": list(decay),
+            "rot": {"base": base, "dims": rot_dims}}
+
+
+def sisepel_dense(ff):
+    return {"kind": "dense", "ff": ff}
+
+
+def sisepel_moe(*, ff, experts, top, shared):
+    mlp = {"kind": "moe", "expert": {"ff": ff}, "router": {"experts": experts, "top": top}}
+    if shared is not None:
+        mlp["shared"] = {"ff": shared}
+    return mlp
+
+
+def sisepel_layer(left, right, mlp=None):
+    return {"type": "parallel", "mixer": {"left": left, "right": right}, "mlp": mlp}
+
+
+def sisepel_config(*, width, vocab, eps, side_dim, logit_scale, layers):
+    cfg = {"architecture": "Sisepel", "width": width, "vocab": vocab, "norm": {"eps": eps},
+           "layers": layers, "logit_scale": logit_scale}
+    if side_dim is not None:
+        cfg["token_side"] = {"dim": side_dim}
+    return cfg
+
+
+# Three small models that differ in every size and option: windows below a page, of several
+# pages, of a single token and none; one key/value head, several, and as many as query heads;
+# value sizes above, below and equal to the key size, on both sides; rotations of two
+# dimensions, of some and of all; frequency scalings that stretch every wave, some and none,
+# and none at all; caps that bend nearly every score, hardly any, and none; decays of one,
+# close to one, of a half and of zero; dense and routed feed-forwards and none; one expert of
+# two and all of them; shared experts wider and narrower than the others and none; models with
+# and without a side input; factors on the logits below, above and equal to one.
+SISE_A = sisepel_config(
+    width=40, vocab=97, eps=1e-5, side_dim=6, logit_scale=0.25, layers=[
+        sisepel_layer(
+            sisepel_attention(heads=4, kv_heads=2, dim=12, vdim=20, scale=0.9, window=3, softcap=1.5,
+                              base=10000.0, rot_dims=8, scaling=sisepel_scaling(3.0, 1.0, 4.0, 40)),
+            sisepel_retention(dim=8, vdim=12, decay=(0.5, 0.97, 1.0), base=500.0, rot_dims=8),
+            sisepel_dense(24)),
+        sisepel_layer(
+            sisepel_attention(heads=3, kv_heads=3, dim=16, vdim=6, scale=1.3, window=18, softcap=20.0,
+                              base=300.0, rot_dims=16, scaling=sisepel_scaling(8.0, 2.0, 3.0, 1000)),
+            sisepel_retention(dim=20, vdim=5, decay=(0.9,), base=100.0, rot_dims=6),
+            sisepel_moe(ff=12, experts=6, top=2, shared=20)),
+        sisepel_layer(
+            sisepel_attention(heads=2, kv_heads=1, dim=6, vdim=10, scale=2.0, window=7, softcap=None,
+                              base=50.0, rot_dims=2),
+            sisepel_retention(dim=4, vdim=16, decay=(0.0, 0.999), base=1e6, rot_dims=2), None),
+    ])
+SISE_B = sisepel_config(
+    width=72, vocab=131, eps=3e-6, side_dim=16, logit_scale=1.0, layers=[
+        sisepel_layer(
+            sisepel_attention(heads=6, kv_heads=1, dim=24, vdim=16, scale=0.7, window=37, softcap=5.0,
+                              base=1e5, rot_dims=12, scaling=sisepel_scaling(4.0, 1.5, 1.5, 64)),
+            sisepel_retention(dim=16, vdim=24, decay=(0.8, 0.99, 0.96875, 0.9995), base=1e4, rot_dims=16),
+            sisepel_moe(ff=16, experts=5, top=5, shared=None)),
+        sisepel_layer(
+            sisepel_attention(heads=5, kv_heads=5, dim=8, vdim=8, scale=1.1, window=None, softcap=2.0,
+                              base=1e4, rot_dims=8),
+            sisepel_retention(dim=10, vdim=10, decay=(0.98, 0.9375), base=1e4, rot_dims=4), None),
+        sisepel_layer(
+            sisepel_attention(heads=4, kv_heads=2, dim=32, vdim=32, scale=0.5, window=50, softcap=30.0,
+                              base=2000.0, rot_dims=20, scaling=sisepel_scaling(2.0, 1.0, 8.0, 100000)),
+            sisepel_retention(dim=32, vdim=8, decay=(0.995, 0.9), base=1e5, rot_dims=8),
+            sisepel_moe(ff=8, experts=2, top=1, shared=4)),
+        sisepel_layer(
+            sisepel_attention(heads=1, kv_heads=1, dim=16, vdim=40, scale=1.4, window=16, softcap=8.0,
+                              base=700.0, rot_dims=4, scaling=sisepel_scaling(5.0, 1.0, 2.0, 4)),
+            sisepel_retention(dim=6, vdim=9, decay=(0.9921875,), base=300.0, rot_dims=6),
+            sisepel_dense(56)),
+    ])
+SISE_C = sisepel_config(
+    width=32, vocab=64, eps=1e-4, side_dim=None, logit_scale=2.5, layers=[
+        sisepel_layer(
+            sisepel_attention(heads=8, kv_heads=4, dim=16, vdim=16, scale=0.8, window=1, softcap=3.0,
+                              base=1e4, rot_dims=16, scaling=sisepel_scaling(16.0, 1.0, 4.0, 256)),
+            sisepel_retention(dim=12, vdim=12, decay=(0.99, 0.75), base=1e4, rot_dims=10),
+            sisepel_moe(ff=20, experts=9, top=3, shared=8)),
+        sisepel_layer(
+            sisepel_attention(heads=2, kv_heads=2, dim=8, vdim=32, scale=1.5, window=64, softcap=12.0,
+                              base=100.0, rot_dims=6, scaling=sisepel_scaling(2.0, 0.5, 1.0, 30)),
+            sisepel_retention(dim=8, vdim=32, decay=(0.96, 0.998, 0.25), base=60.0, rot_dims=8),
+            sisepel_dense(20)),
+    ])
+SISE = {"A": (SISE_A, 85, 4), "B": (SISE_B, 84, 16), "C": (SISE_C, 83, 8)}   # cfg, seed, page
+
+
+def write_sisepel_model(folder, cfg, seed, dtype, std=0.2, router=4.0):
+    """Random weights, with the router's scaled up (`router`), so that the experts' logits lie
+    apart and no choice is decided by rounding.  (Queries and keys are normed: how sharp the
+    attention is is given by its scale and its cap.)"""
+    from safetensors.torch import load_file, save_file
+    from tokensprint_amd.weights import write_random_model
+    d = write_random_model(folder, cfg, seed, dtype, std=std)
+    file = next(d.glob("*.safetensors"))
+    tensors = load_file(str(file))
+    for name in tensors:
+        if name.endswith(".mlp.router"):
+            tensors[name] = (tensors[name].float() * router).to(tensors[name].dtype)
+    save_file(tensors, str(file))
+    return d

@@ -60,6 +60,7 @@ __host__ __device__ __forceinline__ bool has_score_extras(const AttentionArgs& a
 // What turns a query row's products into scores, when there are such extras.
 struct ScoreExtra {
   int pos;                // the query's position (distances are counted from it)
+  bool sloped;            // whether there is a distance bias (the same for all rows)
   float row_scale;        // scale times the query's temperature
   float cap, inv_cap;     // cap 0: none
   float slope;            // of the row's head; 0: none
@@ -74,24 +75,49 @@ __device__ __forceinline__ ScoreExtra score_extra(const AttentionArgs& a, int he
   x.row_scale = a.scale * temp;
   x.cap = a.softcap;
   x.inv_cap = a.softcap > 0.f ? 1.f / a.softcap : 0.f;
+  x.sloped = a.slopes != nullptr;
   x.slope = (a.slopes && pos >= 0) ? a.slopes[head] : 0.f;
   return x;
 }
 
-// A score from the product q . k for the key at position `key`.  FAST: the hyperbolic
-// tangent as 1 - 2 / (exp(2 z) + 1) by the hardware's exponential and reciprocal (for
-// kernels whose operands are bfloat16; the float32 kernel takes the library's).
-template <bool FAST = false>
+// A score from the product q . k for the key at position `key` (the float32 kernel's form).
 __device__ __forceinline__ float extra_score(const ScoreExtra& x, float dot, int key) {
   float s = dot * x.row_scale;
-  if (x.cap > 0.f) {
-    const float z = s * x.inv_cap;
-    const float th = FAST ? 1.f - 2.f * __builtin_amdgcn_rcpf(
-                                      __builtin_amdgcn_exp2f(fminf(z * 2.88539008177792681f, 126.f)) + 1.f)
-                          : tanhf(z);
-    s = x.cap * th;
-  }
+  if (x.cap > 0.f) s = x.cap * tanhf(s * x.inv_cap);
   return s - x.slope * (float)(x.pos - key);
+}
+
+// The same in units of log2, for kernels whose operands are bfloat16, in two steps so that a
+// block's scores meet each condition (the same for all rows) once: the cap, its hyperbolic
+// tangent as 1 - 2 / (exp(2 z) + 1) by the hardware's exponential and reciprocal (an
+// infinite exponential gives the cap itself), and what the distance takes off.
+struct ScoreExtraLog2 {
+  float row;              // product -> score
+  float in, cap, fall;    // product -> exponent; the cap; minus twice the cap
+  float slope;
+  int pos;
+  bool capped, sloped;
+};
+
+__device__ __forceinline__ ScoreExtraLog2 in_log2(const ScoreExtra& x) {
+  constexpr float kLog2e = 1.44269504088896341f;
+  return ScoreExtraLog2{x.row_scale * kLog2e, x.row_scale * x.inv_cap * (2.f * kLog2e),
+                        x.cap * kLog2e, -2.f * x.cap * kLog2e, x.slope * kLog2e,
+                        x.pos, x.cap > 0.f, x.sloped};
+}
+
+__device__ __forceinline__ float capped_log2(const ScoreExtraLog2& x, float dot) {
+  return fmaf(x.fall, __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(dot * x.in) + 1.f), x.cap);
+}
+
+__device__ __forceinline__ float off_by_distance(const ScoreExtraLog2& x, float s, int key) {
+  return fmaf(x.slope, (float)(key - x.pos), s);
+}
+
+// One score, both steps.
+__device__ __forceinline__ float extra_score_log2(const ScoreExtraLog2& x, float dot, int key) {
+  const float s = x.capped ? capped_log2(x, dot) : dot * x.row;
+  return x.sloped ? off_by_distance(x, s, key) : s;
 }
 
 // The sum of a row's softmax weights with the head's sink in it.  `m_log2` is the row's

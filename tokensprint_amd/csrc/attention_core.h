@@ -241,7 +241,7 @@ __device__ __forceinline__ void load_query(TileState<HD>& t, const bf16_t* qrow,
 template <int HD, bool LAZY = false, bool PERM = false, bool EXTRA = false>
 __device__ __forceinline__ void tile_update(TileState<HD>& t, const KvBlock<HD>& b, int kb,
                                             float scale_log2, bool interior, int g,
-                                            const ScoreExtra* x = nullptr) {
+                                            const ScoreExtraLog2* x = nullptr) {
   constexpr int KS = TileState<HD>::KS, DB = TileState<HD>::DB;
   f32x4 st[2];
 #pragma unroll
@@ -252,13 +252,23 @@ __device__ __forceinline__ void tile_update(TileState<HD>& t, const KvBlock<HD>&
       st[blk] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(b.k[blk][s], t.q[s], st[blk], 0, 0, 0);
   }
   if (EXTRA) {
+    if (x->capped) {
 #pragma unroll
-    for (int blk = 0; blk < 2; ++blk)
+      for (int j = 0; j < 2; ++j)
 #pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        const int key = PERM ? kb + g * 8 + blk * 4 + i : kb + blk * 16 + g * 4 + i;
-        st[blk][i] = extra_score<true>(*x, st[blk][i], key) * 1.44269504088896341f;
-      }
+        for (int i = 0; i < 4; ++i) st[j][i] = capped_log2(*x, st[j][i]);
+    } else {
+#pragma unroll
+      for (int j = 0; j < 2; ++j)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) st[j][i] *= x->row;
+    }
+    if (x->sloped) {
+#pragma unroll
+      for (int j = 0; j < 2; ++j)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) st[j][i] = off_by_distance(*x, st[j][i], PERM ? kb + g * 8 + j * 4 + i : kb + j * 16 + g * 4 + i);
+    }
     scale_log2 = 1.f;
   }
   if (!interior) {

@@ -234,8 +234,8 @@ __global__ __launch_bounds__(decode_waves<HD>() * kWave) void attention_decode_k
   t.lo = lo;
   t.keep = a.keep;
   const float scale_log2 = a.scale * 1.44269504088896341f;
-  ScoreExtra x;
-  if (EXTRA) x = score_extra(a, head, row_ok ? pos : -1);   // distances from the query's own position
+  ScoreExtraLog2 x;
+  if (EXTRA) x = in_log2(score_extra(a, head, row_ok ? pos : -1));   // distances from the query's own position
   const int stride = walkers * 32;
   const int key_begin = max(c0 * kChunk, walk.origin) + wave * 32;
   const int key_end = (prep_wave || key_wave) ? 0 : min(c1 * kChunk, last + 1);
@@ -283,7 +283,7 @@ __global__ __launch_bounds__(decode_waves<HD>() * kWave) void attention_decode_k
 #pragma unroll
         for (int j = 0; j < 8; ++j) dot += (float)t.q[s][j] * (float)kq[s][j];
       // this wave's partial: one key with weight 1
-      t.m = EXTRA ? extra_score<true>(x, col4_sum(dot), pos) * 1.44269504088896341f
+      t.m = EXTRA ? extra_score_log2(x, col4_sum(dot), pos)
                   : col4_sum(dot) * scale_log2;
       t.l = g == 0 ? 1.f : 0.f;
 #pragma unroll

@@ -58,8 +58,8 @@ __global__ __launch_bounds__(256, HD <= 128 ? 2 : 1) void attention_mfma_kernel(
   t.keep = a.keep;
   load_query<HD>(t, (const bf16_t*)a.q + ((int64_t)token * a.nq + head) * HD, row_ok, g);
   const float scale_log2 = a.scale * 1.44269504088896341f;
-  ScoreExtra x;
-  if (EXTRA) x = score_extra(a, head, t.pos);
+  ScoreExtraLog2 x;
+  if (EXTRA) x = in_log2(score_extra(a, head, t.pos));
   const int lo_last = first_visible(a, pos_last);
 
   constexpr int kStride = COOP ? 128 : 32;

@@ -380,7 +380,7 @@ __global__ __launch_bounds__(256 * H, H == 1 ? 3 : 2) void attention_prefill_asy
 template <int HD, bool DEEP, bool EXTRA, typename Between>
 __device__ __forceinline__ void tile_update64(TileState<HD>& t, bf16x8 (*buf)[kWave], int lane, int kb,
                                               float scale_log2, bool interior, int g,
-                                              Between between, const ScoreExtra* x = nullptr) {
+                                              Between between, const ScoreExtraLog2* x = nullptr) {
   constexpr int KS = HD / 32, DB = HD / 16, kSlots = 2 * KS + DB;
   f32x4 st[4];
 #pragma unroll
@@ -418,13 +418,23 @@ __device__ __forceinline__ void tile_update64(TileState<HD>& t, bf16x8 (*buf)[kW
     __builtin_amdgcn_sched_barrier(0);
   }
   if (EXTRA) {
+    if (x->capped) {
 #pragma unroll
-    for (int j = 0; j < 4; ++j)
+      for (int j = 0; j < 4; ++j)
 #pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        const int key = kb + (j / 2) * 32 + g * 8 + (j % 2) * 4 + i;
-        st[j][i] = extra_score<true>(*x, st[j][i], key) * 1.44269504088896341f;
-      }
+        for (int i = 0; i < 4; ++i) st[j][i] = capped_log2(*x, st[j][i]);
+    } else {
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) st[j][i] *= x->row;
+    }
+    if (x->sloped) {
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) st[j][i] = off_by_distance(*x, st[j][i], kb + (j / 2) * 32 + g * 8 + (j % 2) * 4 + i);
+    }
     scale_log2 = 1.f;
   }
   if (!interior) {
@@ -584,8 +594,8 @@ __device__ __forceinline__ void attention_prefill_wide(const AttentionMfmaArgs& 
     t.pos = row_ok ? pos_first + ti : -1;
     t.lo = first_visible(a, t.pos);
     t.keep = a.keep;
-    ScoreExtra x;
-    if (EXTRA) x = score_extra(a, head, t.pos);
+    ScoreExtraLog2 x;
+    if (EXTRA) x = in_log2(score_extra(a, head, t.pos));
     const int tile_first = pos_first + wave * tq;
     const int tile_last = wave * tq < ntok ? pos_first + min(ntok, (wave + 1) * tq) - 1 : -1;
     const int tile_lo = first_visible(a, tile_first);

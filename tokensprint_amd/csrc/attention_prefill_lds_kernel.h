@@ -57,8 +57,8 @@ __global__ __launch_bounds__(256, HD <= 128 ? 4 : 1) void attention_prefill_lds_
   t.pos = row_ok ? pos_first + ti : -1;
   t.lo = first_visible(a, t.pos);
   t.keep = a.keep;
-  ScoreExtra x;
-  if (EXTRA) x = score_extra(a, head, t.pos);
+  ScoreExtraLog2 x;
+  if (EXTRA) x = in_log2(score_extra(a, head, t.pos));
   const int tile_first = pos_first + wave * tq;
   const int tile_last = wave * tq < ntok ? pos_first + min(ntok, (wave + 1) * tq) - 1 : -1;
   const int tile_lo = first_visible(a, tile_first);
