@@ -131,3 +131,25 @@ def test_fubepel_and_zonopel_are_compared_at_equal_size():
         assert len(fube["layers"]) == len(zono["layers"])
         assert {e["type"] for e in fube["layers"]} == {"latent_attention", "delta", "attention"}
         assert any("kv_from" in e["mixer"] for e in fube["layers"]) and fube["token_side"]
+
+
+def test_sisepel_and_palelix_are_compared_at_equal_size():
+    """`bench.py --compare-sisepel` builds a Sisepel and a Palelix configuration per size with
+    the same width, depth, vocabulary and (within 2 %) number of parameters, every option and
+    both kinds of feed-forward, and retention of the size of the other's linear attention."""
+    import math
+
+    import bench
+    from tokensprint_amd.weights.random_init import declared_tensors
+    for name, size in bench.COMPARE_SIZES.items():
+        sise, pale = bench.sisepel_configs(size)
+        count = [sum(math.prod(d.shape) for d in declared_tensors(raw).values())
+                 for raw in (sise, pale)]
+        assert abs(count[0] - count[1]) <= 0.02 * count[0], (name, count)
+        assert sise["width"] == pale["width"] and sise["vocab"] == pale["vocab"]
+        assert len(sise["layers"]) == len(pale["layers"])
+        assert {e["mlp"]["kind"] for e in sise["layers"]} == {"dense", "moe"}
+        left, right = (sise["layers"][1]["mixer"][side] for side in ("left", "right"))
+        assert {"softcap", "mask", "rot"} <= set(left) and sise["token_side"]
+        other = next(e["mixer"] for e in pale["layers"] if e["type"] == "lightning")
+        assert [right[k] for k in ("heads", "dim", "vdim")] == [other[k] for k in ("heads", "dim", "vdim")]

@@ -222,3 +222,23 @@ def test_run_py_serves_a_fubepel_model(gpu_device, tmp_path):
     for _ in range(9):
         tokens.append(int(fubepel_plain.forward(pcfg, w, tokens)[-1].argmax()))
     assert got == tokens[len(prompt):]
+
+
+def test_run_py_serves_a_sisepel_model(gpu_device, tmp_path):
+    """The same for Sisepel: windowed attention beside retention, experts with a shared one, a
+    side input of every token, a factor on the logits."""
+    from helpers import SISE_A
+    from plain import sisepel_plain
+    prompt = random_prompt(21, SISE_A["vocab"], 9)
+    model_dir = tmp_path / "sise-a"
+    proc = run_program(["run.py", "--config-json", config_json(tmp_path, SISE_A),
+                        "--random-weights", "2", "--model-dir", model_dir, "--dtype", "float32",
+                        "--temperature", "0", "--max-tokens", "9", "--ignore-eos", "True",
+                        "--max-num-seqs", "8", "--max-model-len", "256",
+                        "--prompt-ids", ",".join(map(str, prompt))])
+    got = json.loads(proc.stdout.strip().splitlines()[-1])
+    pcfg, w = sisepel_plain.read_model_dir(model_dir)
+    tokens = list(prompt)
+    for _ in range(9):
+        tokens.append(int(sisepel_plain.forward(pcfg, w, tokens)[-1].argmax()))
+    assert got == tokens[len(prompt):]

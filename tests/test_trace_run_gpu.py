@@ -14,10 +14,12 @@ import pytest
 import torch
 
 from drives import row_tolerance
-from helpers import (FUBE, PALE, PINE, TINY, ZOLO, ZONO, random_prompt, write_fubepel_model,
-                     write_palelix_model, write_pinedra_model, write_zolorax_model)
+from helpers import (FUBE, PALE, PINE, SISE, TINY, ZOLO, ZONO, random_prompt, write_fubepel_model,
+                     write_palelix_model, write_pinedra_model, write_sisepel_model,
+                     write_zolorax_model)
 from plain import qwen3_plain as plain
-from plain import fubepel_plain, palelix_plain, pinedra_plain, zolorax_plain, zonopel_plain
+from plain import (fubepel_plain, palelix_plain, pinedra_plain, sisepel_plain, zolorax_plain,
+                   zonopel_plain)
 from tokensprint_amd.weights import write_random_model
 
 pytestmark = pytest.mark.gpu
@@ -75,7 +77,8 @@ def check(got, ref, rtol, atol, what):
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
 @pytest.mark.parametrize("name", ["B", "C", "zonopel-A", "zonopel-B", "palelix-A", "palelix-B",
                                   "zolorax-A", "zolorax-B", "pinedra-A", "pinedra-B",
-                                  "fubepel-A", "fubepel-B", "fubepel-C"])
+                                  "fubepel-A", "fubepel-B", "fubepel-C", "sisepel-A", "sisepel-B",
+                                  "sisepel-C"])
 def test_replay_variants(tmp_path, name, dtype):
     stored = torch.float32 if dtype == "float32" else torch.bfloat16
     rtol, atol = TOL[dtype]
@@ -125,6 +128,16 @@ def test_replay_variants(tmp_path, name, dtype):
         pcfg, w = fubepel_plain.read_model_dir(model_dir)
         vocab = cfg["vocab"]
         forward = lambda t: fubepel_plain.forward(pcfg, w, t).float()
+        rtol, atol = max(rtol, 2e-4), max(atol, 1e-4)
+    elif name.startswith("sisepel-"):
+        if dtype == "bfloat16":
+            pytest.skip("this design's bfloat16 runs are judged by a row's root mean square, in "
+                        "test_sisepel_gpu.py")
+        cfg, seed, _ = SISE[name[-1]]
+        model_dir = write_sisepel_model(tmp_path / "model", cfg, seed, stored)
+        pcfg, w = sisepel_plain.read_model_dir(model_dir)
+        vocab = cfg["vocab"]
+        forward = lambda t: sisepel_plain.forward(pcfg, w, t).float()
         rtol, atol = max(rtol, 2e-4), max(atol, 1e-4)
     else:
         cfg, seed, _ = TINY[name]
